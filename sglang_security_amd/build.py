@@ -21,6 +21,8 @@ LIB = os.path.join(PKG, "libsglk.so")
 TORCH_SRC = os.path.join(CSRC, "torch", "allreduce_ops.cc")
 TORCH_LIB = os.path.join(PKG, "sgl_kernel", "common_ops.so")
 ARCH = "gfx950"
+# no packed fp32 vector instructions: some of their forms have given wrong results on these devices
+CODEGEN = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def _hipcc() -> str:
@@ -43,7 +45,7 @@ def _compile(src: str, force: bool) -> str:
     obj = os.path.join(OBJ, os.path.basename(src) + ".o")
     if (not force and os.path.exists(obj) and os.path.getmtime(obj) >= max(os.path.getmtime(src), _deps_mtime())):
         return obj
-    cmd = [_hipcc(), f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-fvisibility=hidden",
+    cmd = [_hipcc(), f"--offload-arch={ARCH}", *CODEGEN, "-O3", "-std=c++17", "-fPIC", "-fvisibility=hidden",
            "-I" + os.path.join(ROOT, "include"), "-I" + CSRC, "-c", src, "-o", obj]
     if src.endswith(".cpp"):
         cmd.insert(1, "-x")

@@ -1475,6 +1475,11 @@ static int ensure_lds(int bytes) {
   return SGLK_OK;
 }
 
+__global__ void __launch_bounds__(256) clear_words_kernel(uint32_t* p, int n) {
+  const int i = blockIdx.x * 256 + threadIdx.x;
+  if (i < n) p[i] = 0;
+}
+
 // Everything the entry point would otherwise do on its first call on a device: the array's address and the LDS
 // limits of every kernel the call can dispatch to.
 template <typename T>
@@ -1866,7 +1871,9 @@ int sglk_awq_gemm_static(const void* x, const int32_t* packed, const void* scale
   const int rc = static_scratch(&ws, out, (hipStream_t)stream, true);
   if (rc != SGLK_OK) return rc;
   // the array keeps the previous call's contents: the ticket words must start at zero
-  SGLK_HIP(hipMemsetAsync(ws, 0, (size_t)kMaxTiles * 4, (hipStream_t)stream));
+  // (a kernel, not a memset node: replays of captured memset nodes are not reliable)
+  hipLaunchKernelGGL(clear_words_kernel, dim3((kMaxTiles + 255) / 256), dim3(256), 0, (hipStream_t)stream,
+                     reinterpret_cast<uint32_t*>(ws), kMaxTiles);
   return sglk_awq_gemm_xs(x, packed, scales, qzeros, bias, out, reinterpret_cast<float*>(ws), M, N, K, group_size,
                           x_stride, out_stride, dtype, nullptr, 0, stream);
 }

@@ -2,7 +2,7 @@
 // 512 threads per block = 2 waves per SIMD, one block per CU.  Per iteration a wave issues 16 MFMAs
 // (16 independent accumulators) and / or 48 integer VALU instructions shaped like the int4 dequantisation
 // (shift, and-or), in blocks of 4 MFMA + 12 VALU.
-// build: hipcc --offload-arch=gfx950 -O3 tools/coissue.hip -o tools/coissue.bin
+// build: hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 tools/coissue.hip -o tools/coissue.bin
 #include <hip/hip_runtime.h>
 #include <cstdio>
 typedef float float4v __attribute__((ext_vector_type(4)));

@@ -1,7 +1,7 @@
 // Micro-benchmark: cost of a grid-wide barrier between co-resident blocks (one agent-scope counter, bounded polling),
 // with and without a release / acquire fence pair around it, next to the cost of a dependent kernel boundary.
 // Every poll loop is bounded and watches an abort word, so the grid drains even if a block never arrives.
-// build: hipcc --offload-arch=gfx950 -O3 tools/gridbar.hip -o gpurun_out/gridbar
+// build: hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 tools/gridbar.hip -o gpurun_out/gridbar
 #include <hip/hip_runtime.h>
 #include <cstdio>
 

@@ -2,7 +2,7 @@
 // independent loads in flight per lane):  read-only sweep, read-only sweep with non-temporal loads, and copy.
 // Buffers are far larger than the 256 MiB Infinity Cache.  Prints one JSON line.
 //
-//   hipcc --offload-arch=gfx950 -O3 -o tools/hbm_probe.bin tools/hbm_probe.hip && tools/hbm_probe.bin [GiB]
+//   hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -o tools/hbm_probe.bin tools/hbm_probe.hip && tools/hbm_probe.bin [GiB]
 #include <hip/hip_runtime.h>
 
 #include <cstdio>
