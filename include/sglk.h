@@ -996,6 +996,103 @@ SGLK_API int64_t sglk_radix_node_key(int64_t tree, int64_t node, int32_t* key_ou
 /* pre-order dump, children ordered by first token: per node 12 int64 fields (see sglk_radix_node_get) */
 SGLK_API int64_t sglk_radix_dump(int64_t tree, int64_t* node_ids, int64_t cap);
 
+/* ------------------------------------------------- decoders with an fp32 residual stream, latent attention and gated
+ * linear recurrences.  A "source" (src, src_f32, splits, part_stride, src_stride) is a product's result: src_f32 = 1 the
+ * fp32 split sums partial[split][row][col] (part_stride floats from split to split), added up in split order by the
+ * consumer; src_f32 = 0 finished rows of the activation type.  Rows are padded to multiples of eight elements, zeros
+ * in the padding. */
+
+/* One block per row.  x = embed[ids[row]] * embed_scale (embed != NULL; also stored to x0 if that is given) or the
+ * residual row as it is; x += norm(src) * w_post (src != NULL; added as it is without w_post); x += x0 (add_x0);
+ * x += step (step != NULL); stored back if store_x; h = norm(x) * w_next (w_next != NULL).  norm(v) = v / sqrt(mean(v^2) +
+ * eps) over `width` elements.  rows != NULL: output row r works on row rows[r]. */
+SGLK_API int sglk_residual_norm(float* x, const void* embed, const int32_t* ids, int64_t embed_stride, float embed_scale,
+                                const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
+                                const float* w_post, float* x0, int add_x0, const float* step, const float* w_next, void* h,
+                                int64_t h_stride, const int32_t* rows, int store_x, int M, int width, int pitch, float eps,
+                                int dtype, void* stream);
+/* out[m][n] = act(src[m][n] + bias[n]); act: 0 none, 1 square of relu, 2 gelu (tanh form) */
+SGLK_API int sglk_source_act(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
+                             const float* bias, void* out, int M, int N, int64_t out_stride, int act, int dtype,
+                             void* stream);
+/* fp32 logits [M, V] = cap * tanh(src / cap) (cap <= 0: src) */
+SGLK_API int sglk_capped_logits(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
+                                float* out, int M, int N, int V, int64_t out_stride, float cap, int dtype, void* stream);
+/* req_to_token[req[row_seq[t]]][positions[t]] = loc[t] */
+SGLK_API int sglk_assign_slots(int32_t* req_to_token, int64_t row_stride, const int32_t* row_seq, const int32_t* req,
+                               const int32_t* positions, const int32_t* loc, int T, void* stream);
+
+/* Latent attention; a pool row is [latent, r_pitch | rotated key part, rot_pitch].
+ * latent_prep: src columns [q_pitch query latent | r_pitch latent | rot_pitch rotated part] -> cq (normalised), pool rows
+ * loc[m] (normalised latent, rotation by cos_sin[position] = cos[rot_dims / 2] | sin[rot_dims / 2]). */
+SGLK_API int sglk_latent_prep(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
+                              const float* wq, const float* wkv, void* cq, int64_t cq_stride, void* pool,
+                              int64_t pool_stride, const int32_t* loc, const float* cos_sin, const int32_t* positions, int M,
+                              int q_rank, int q_pitch, int kv_rank, int r_pitch, int rot_dim, int rot_pitch, int rot_dims,
+                              float eps, int dtype, void* stream);
+SGLK_API int sglk_latent_rope_q(const void* src, int64_t src_m, int64_t src_h, void* out, int64_t out_m, int64_t out_h,
+                                const float* cos_sin, const int32_t* positions, int M, int H, int rot_pitch, int rot_dims,
+                                int dtype, void* stream);
+/* out[m][h][n] = sum_k a[m][h][k] w[h][n][k].  bf16: w in operand order [H][Np / 16][K / 32][64 lanes][8] (lane 16 g + i:
+ * column 16 s + i, k = 32 ks + 8 g + e); other types: row-major [H][Np][K].  lse != NULL: a holds the split partials
+ * [M][H][splits][K] (fp32) of sglk_latent_decode, merged first. */
+SGLK_API int sglk_head_gemm(const void* a, const float* lse, int splits, int64_t a_m, int64_t a_h, const void* w, void* out,
+                            int M, int H, int N, int Np, int K, int64_t out_m, int64_t out_h, int dtype, void* stream);
+SGLK_API int sglk_latent_decode_supported(int r_pitch, int rot_pitch);
+/* bf16 rows of one token each: q [M, H, r_pitch + rot_pitch] against the pool rows of positions (p - window, p] of request
+ * req[m] (window <= 0: [0, p]); leaves `splits` normalised partials part [M][H][splits][r_pitch] and their
+ * log-sum-exps (-inf: empty split). */
+SGLK_API int sglk_latent_decode(const void* q, int64_t q_m, int64_t q_h, const void* pool, int64_t pool_stride,
+                                const int32_t* req_to_token, int64_t r2t_stride, const int32_t* req,
+                                const int32_t* positions, float* part, float* lse, int M, int H, int r_pitch, int rot_pitch,
+                                int window, int splits, float scale, void* stream);
+/* the same, finished rows out [M, H, DV], any size and float type (one wave per row and head) */
+SGLK_API int sglk_latent_attention_rows(const void* q, int64_t q_m, int64_t q_h, const void* pool, int64_t pool_stride,
+                                        const int32_t* req_to_token, int64_t r2t_stride, const int32_t* req,
+                                        const int32_t* positions, void* out, int64_t out_m, int64_t out_h, int M, int H,
+                                        int D, int DV, int window, float scale, int dtype, void* stream);
+SGLK_API int sglk_latent_prefill_supported(int k_pitch, int v_pitch);
+/* bf16 runs of rows: sequence b has rows[b] query rows from row0[b] on and sees the tokens from tok0[b] on of k / v / kr
+ * (expanded keys and values, shared rotated key parts of 64 elements); its row i stands at token ahead[b] + i. */
+SGLK_API int sglk_latent_prefill(const void* q, int64_t q_m, const void* k, int64_t k_n, const void* v, int64_t v_n,
+                                 const void* kr, int64_t kr_n, void* o, int64_t o_m, int64_t o_h, const int32_t* row0,
+                                 const int32_t* rows, const int32_t* tok0, const int32_t* ahead, int n_seqs, int max_rows,
+                                 int H, int k_pitch, int v_pitch, int vdim, int window, float scale, void* stream);
+
+/* Gated linear recurrence behind a causal convolution (rglru.hip): src columns [W x branch | W y branch], channels stored
+ * block by block with bwp per block; conv [taps][W]; conv_state [slots][taps - 1][W] of the activation type; state [slots][W]
+ * fp32.  Sequences: row_seq per row; row0, rows, start, slot per sequence; the first `singles` rows are sequences of one
+ * row. */
+SGLK_API int sglk_rglru_conv(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
+                             const float* bx, const float* by, const float* conv, const float* conv_b, void* u, void* y,
+                             void* conv_state, const int32_t* row_seq, const int32_t* row0, const int32_t* rows,
+                             const int32_t* start, const int32_t* slot, int M, int W, int taps, int singles, int n_seqs,
+                             int dtype, void* stream);
+/* gate weights wr, wi (bf16) in operand order [blocks][bwp / 16][bwp / 32][64 lanes][8]; sp = softplus(lambda) */
+SGLK_API int sglk_rglru_step(const void* u, const void* wr, const void* wi, const float* br, const float* bi,
+                             const float* sp, const void* y, float* state, const int32_t* start, const int32_t* slot,
+                             void* out, int64_t out_stride, int M, int W, int bwp, int blocks, void* stream);
+SGLK_API int sglk_rglru_gates(const void* u, const void* wr, const void* wi, const float* br, const float* bi,
+                              const float* sp, const int32_t* tile_row, const int32_t* tile_rows, int tiles, float* hloc,
+                              float* prod, int W, int bwp, int blocks, void* stream);
+SGLK_API int sglk_rglru_carry(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
+                              const float* bx, const float* by, const float* conv, const float* conv_b, void* u, void* y,
+                              void* conv_state, const int32_t* row_seq, const int32_t* row0, const int32_t* rows,
+                              const int32_t* start, const int32_t* slot, int M, int W, int taps, int singles, int n_seqs,
+                              const float* hloc, const float* prod, float* carry, float* state, const int32_t* tile0,
+                              int seq0, int used, int dtype, void* stream);
+SGLK_API int sglk_rglru_apply(const float* hloc, const float* prod, const float* carry, const void* y, void* out,
+                              int64_t out_stride, const int32_t* row_seq, const int32_t* row0, const int32_t* tile0,
+                              int first_row, int M, int W, int used, int dtype, void* stream);
+/* any type and block size; gate weights row-major [blocks][bwp][bwp] */
+SGLK_API int sglk_rglru_rows(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
+                             const float* bx, const float* by, const float* conv, const float* conv_b, void* u, void* y,
+                             void* conv_state, const int32_t* row_seq, const int32_t* row0, const int32_t* rows,
+                             const int32_t* start, const int32_t* slot, int M, int W, int taps, int singles, int n_seqs,
+                             const void* wr, const void* wi, const float* br, const float* bi, const float* sp, float* da,
+                             float* db, float* state, void* out, int64_t out_stride, int bwp, int blocks, int dtype,
+                             void* stream);
+
 #ifdef __cplusplus
 }
 #endif

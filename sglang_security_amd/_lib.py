@@ -129,6 +129,32 @@ _SIGS = {
     "sglk_awq_chain_sync_bytes": (i64, []),
     "sglk_awq_chain_status": (i32, [p]),
     "sglk_awq_chain": (i32, [p, i32, p, i32, i32, i32, p]),
+    "sglk_residual_norm": (i32, [p, p, p, i64, f32, p, i32, i32, i64, i64, p, p, i32, p, p, p, i64, p, i32, i32,
+        i32, i32, f32, i32, p]),
+    "sglk_source_act": (i32, [p, i32, i32, i64, i64, p, p, i32, i32, i64, i32, i32, p]),
+    "sglk_capped_logits": (i32, [p, i32, i32, i64, i64, p, i32, i32, i32, i64, f32, i32, p]),
+    "sglk_assign_slots": (i32, [p, i64, p, p, p, p, i32, p]),
+    "sglk_latent_prep": (i32, [p, i32, i32, i64, i64, p, p, p, i64, p, i64, p, p, p, i32, i32, i32, i32, i32,
+        i32, i32, i32, f32, i32, p]),
+    "sglk_latent_rope_q": (i32, [p, i64, i64, p, i64, i64, p, p, i32, i32, i32, i32, i32, p]),
+    "sglk_head_gemm": (i32, [p, p, i32, i64, i64, p, p, i32, i32, i32, i32, i32, i64, i64, i32, p]),
+    "sglk_latent_decode_supported": (i32, [i32, i32]),
+    "sglk_latent_decode": (i32, [p, i64, i64, p, i64, p, i64, p, p, p, p, i32, i32, i32, i32, i32, i32, f32,
+        p]),
+    "sglk_latent_attention_rows": (i32, [p, i64, i64, p, i64, p, i64, p, p, p, i64, i64, i32, i32, i32, i32,
+        i32, f32, i32, p]),
+    "sglk_latent_prefill_supported": (i32, [i32, i32]),
+    "sglk_latent_prefill": (i32, [p, i64, p, i64, p, i64, p, i64, p, i64, i64, p, p, p, p, i32, i32, i32, i32,
+        i32, i32, i32, f32, p]),
+    "sglk_rglru_conv": (i32, [p, i32, i32, i64, i64, p, p, p, p, p, p, p, p, p, p, p, p, i32, i32, i32, i32,
+        i32, i32, p]),
+    "sglk_rglru_step": (i32, [p, p, p, p, p, p, p, p, p, p, p, i64, i32, i32, i32, i32, p]),
+    "sglk_rglru_gates": (i32, [p, p, p, p, p, p, p, p, i32, p, p, i32, i32, i32, p]),
+    "sglk_rglru_carry": (i32, [p, i32, i32, i64, i64, p, p, p, p, p, p, p, p, p, p, p, p, i32, i32, i32, i32,
+        i32, p, p, p, p, p, i32, i32, i32, p]),
+    "sglk_rglru_apply": (i32, [p, p, p, p, p, i64, p, p, p, i32, i32, i32, i32, i32, p]),
+    "sglk_rglru_rows": (i32, [p, i32, i32, i64, i64, p, p, p, p, p, p, p, p, p, p, p, p, i32, i32, i32, i32,
+        i32, p, p, p, p, p, p, p, p, p, i64, i32, i32, i32, p]),
     "sglk_ar_meta_size": (i64, []),
     "sglk_ar_init": (i64, [p, i32, i32, i32, i64]),
     "sglk_ar_init_handles": (i64, [p, p, i64, p, p, i32, i32, i32, i64]),
@@ -179,6 +205,15 @@ class SglkError(RuntimeError):
     TORCH_CHECK in the same situations)."""
 
 
+_partial = False
+
+
+def use_partial(path: str):
+    """Load a library that holds only some of the sources: what it lacks fails when it is called."""
+    global LIB_PATH, _partial
+    LIB_PATH, _partial = path, True
+
+
 def lib():
     global _lib
     if _lib is None:
@@ -190,6 +225,8 @@ def lib():
         L = C.CDLL(LIB_PATH)
         for name, (res, args) in _SIGS.items():
             if name in _PENDING:
+                continue
+            if _partial and not hasattr(L, name):
                 continue
             fn = getattr(L, name)  # AttributeError if the library is stale: fail loudly
             fn.restype = res

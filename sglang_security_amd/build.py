@@ -70,6 +70,36 @@ def build(force: bool = False, jobs: int = 6) -> str:
     return LIB
 
 
+# what the checkpoint-loaded models of the engine launch, and nothing else
+ENGINE = ("core.hip", "elementwise.hip", "gemm_dense.hip", "sampling.hip", "latent_attention.hip", "residual_norm.hip", "rglru.hip")
+
+
+def ensure(names, jobs: int = 8) -> str:
+    """Without a full library beside the package: compile the named sources into a library of their own (once; other
+    processes wait for the one that compiles) and make this process load that."""
+    from . import _lib
+
+    if os.environ.get("SGLK_LIB") or os.path.exists(LIB):
+        return _lib.LIB_PATH
+    import fcntl
+
+    os.makedirs(OBJ, exist_ok=True)
+    part = os.path.join(PKG, "libsglk_engine.so")
+    with open(os.path.join(OBJ, ".lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        with cf.ThreadPoolExecutor(max_workers=jobs) as ex:
+            objs = list(ex.map(lambda n: _compile(os.path.join(CSRC, n), False), names))
+        if not os.path.exists(part) or any(os.path.getmtime(o) > os.path.getmtime(part) for o in objs):
+            tmp = f"{part}.{os.getpid()}"
+            r = subprocess.run([_hipcc(), f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", tmp] + objs, capture_output=True,
+                               text=True)
+            if r.returncode != 0:
+                raise RuntimeError("link failed:\n" + r.stderr)
+            os.replace(tmp, part)
+    _lib.use_partial(part)
+    return part
+
+
 def build_torch_ops(force: bool = False) -> str:
     """sgl_kernel/common_ops.so: the torch.ops.sgl_kernel.* registrations that have to come from C++ (the all-reduce
     op set, whose `str[]` arguments carry raw handle bytes).  Host code only: g++ against the installed torch's

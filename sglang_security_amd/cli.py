@@ -1,0 +1,90 @@
+"""Command line.
+
+    python -m sglang_security_amd.cli models
+    python -m sglang_security_amd.cli generate --model DIR --prompt-ids 1,2,3 [--prompt-ids ...] [--max-new-tokens N]
+        [--temperature T] [--top-k K] [--top-p P] [--min-p P] [--dtype bfloat16|float32] ...
+    python -m sglang_security_amd.cli trace --model DIR --dtype D --out DIR --max-tokens N   (steps on standard input)
+
+`generate` takes prompts as token ids (one --prompt-ids each, or a JSON file of lists with --prompts) and prints one JSON
+line per request: {"id": ..., "output_ids": [...]}.
+"""
+from __future__ import annotations
+
+import argparse
+import json
+import sys
+
+
+def _generate(args) -> int:
+    import torch
+
+    from .engine import Engine, SamplingParams, Scheduler
+    from .models import load_model
+
+    if not torch.cuda.is_available():
+        raise SystemExit("no GPU (there is no CPU fallback)")
+    prompts = [[int(t) for t in p.replace(",", " ").split()] for p in args.prompt_ids or []]
+    if args.prompts:
+        with open(args.prompts) as f:
+            prompts += json.load(f)
+    if not prompts:
+        raise SystemExit("no prompts")
+    params = SamplingParams(args.max_new_tokens, args.temperature, args.top_k, args.top_p, args.min_p, tuple(args.stop or ()))
+    dev = torch.device("cuda", args.device)
+    torch.cuda.set_device(dev)
+    longest = max(len(p) for p in prompts) + args.max_new_tokens
+    context = args.max_context or longest
+    model = load_model(args.model, getattr(torch, args.dtype), dev, context)
+    engine = Engine(model, args.max_tokens or context * min(len(prompts), args.max_requests), args.max_requests,
+                    use_graph=not args.no_graph)
+    for i, out in enumerate(Scheduler(engine, args.prefill_budget, args.seed).generate(prompts, params)):
+        print(json.dumps({"id": i, "output_ids": out}), flush=True)
+    return 0
+
+
+def _models(_args) -> int:
+    from .models import ARCHITECTURES, SYNTHETIC
+
+    for name in sorted(ARCHITECTURES):
+        print(f"{name}\tcheckpoint")
+    for name in sorted(SYNTHETIC):
+        print(f"{name}\tsynthetic (bench.py --model)")
+    return 0
+
+
+def main(argv=None) -> int:
+    argv = sys.argv[1:] if argv is None else argv
+    if argv and argv[0] == "trace":
+        from .trace import main as trace_main
+
+        return trace_main(argv[1:])
+    ap = argparse.ArgumentParser(prog="sglang_security_amd", description=__doc__,
+                                 formatter_class=argparse.RawDescriptionHelpFormatter)
+    sub = ap.add_subparsers(dest="command", required=True)
+    sub.add_parser("models", help="list the model registry").set_defaults(run=_models)
+    sub.add_parser("trace", help="replay a trace of steps (see `trace --help`)")
+    g = sub.add_parser("generate", help="generate from token-id prompts")
+    g.add_argument("--model", required=True, help="folder with config.json and *.safetensors")
+    g.add_argument("--prompt-ids", action="append", help="one prompt: token ids with commas or spaces between them")
+    g.add_argument("--prompts", help="JSON file: a list of lists of token ids")
+    g.add_argument("--max-new-tokens", type=int, default=16)
+    g.add_argument("--temperature", type=float, default=0.0, help="0: greedy")
+    g.add_argument("--top-k", type=int, default=0)
+    g.add_argument("--top-p", type=float, default=1.0)
+    g.add_argument("--min-p", type=float, default=0.0)
+    g.add_argument("--stop", type=int, action="append", help="token id that ends a request")
+    g.add_argument("--seed", type=int, default=0)
+    g.add_argument("--dtype", default="bfloat16", choices=["bfloat16", "float32"])
+    g.add_argument("--max-requests", type=int, default=64, help="live requests at most")
+    g.add_argument("--max-tokens", type=int, default=0, help="slots of the KV pool (default: what the prompts can need)")
+    g.add_argument("--max-context", type=int, default=0)
+    g.add_argument("--prefill-budget", type=int, default=2048, help="prompt tokens per step")
+    g.add_argument("--no-graph", action="store_true")
+    g.add_argument("--device", type=int, default=0)
+    g.set_defaults(run=_generate)
+    args = ap.parse_args(argv)
+    return args.run(args)
+
+
+if __name__ == "__main__":
+    sys.exit(main())

@@ -1459,22 +1459,6 @@ WidePlan plan_awq_wide(int M, int N, int K, int group_size, bool partial_mode) {
 
 using namespace sglk;
 
-static constexpr int kMaxDevices = 64;
-
-// Raises a kernel's dynamic-LDS limit once per (kernel, device): the attribute belongs to the device's copy of the
-// code object.  One flag array per kernel, shared by the launch sites and by sglk_awq_gemm_static_init().
-template <auto Kernel>
-static int ensure_lds(int bytes) {
-  static bool done[kMaxDevices];
-  int dev = 0;
-  SGLK_HIP(hipGetDevice(&dev));
-  if (dev < 0 || dev >= kMaxDevices || !done[dev]) {
-    SGLK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(Kernel), hipFuncAttributeMaxDynamicSharedMemorySize, bytes));
-    if (dev >= 0 && dev < kMaxDevices) done[dev] = true;
-  }
-  return SGLK_OK;
-}
-
 __global__ void __launch_bounds__(256) clear_words_kernel(uint32_t* p, int n) {
   const int i = blockIdx.x * 256 + threadIdx.x;
   if (i < n) p[i] = 0;

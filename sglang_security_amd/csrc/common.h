@@ -280,6 +280,22 @@ __device__ __forceinline__ int64_t ld_idx(const void* p, int is64, int64_t i) {
       return ::sglk::fail(SGLK_EINVAL, "dtype code %d: expected fp16 or bf16", dtype); \
   }
 
+constexpr int kMaxDevices = 64;
+
+// Raises a kernel's dynamic-LDS limit once per (kernel, device): the attribute belongs to the device's copy of the
+// code object.  One flag array per kernel and source file.
+template <auto Kernel>
+inline int ensure_lds(int bytes) {
+  static bool done[kMaxDevices];
+  int dev = 0;
+  SGLK_HIP(hipGetDevice(&dev));
+  if (dev < 0 || dev >= kMaxDevices || !done[dev]) {
+    SGLK_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(Kernel), hipFuncAttributeMaxDynamicSharedMemorySize, bytes));
+    if (dev >= 0 && dev < kMaxDevices) done[dev] = true;
+  }
+  return SGLK_OK;
+}
+
 inline int elem_size(int dtype) { return dtype == SGLK_F32 ? 4 : (dtype == SGLK_FP8_E4M3 ? 1 : 2); }
 
 }  // namespace sglk

@@ -204,3 +204,38 @@ class MLATokenToKVPool:
         """memory_pool.py:613-625 (set_mla_kv_buffer_triton :446-508): the row is [nope | rope]."""
         row = torch.cat([cache_k_nope.reshape(loc.numel(), -1), cache_k_rope.reshape(loc.numel(), -1)], dim=-1)
         self.set_kv_buffer(layer, loc, row, row)
+
+
+class RecurrentStatePool:
+    """State of one recurrent layer: per slot the fp32 recurrence state and the last taps - 1 inputs of its convolution.
+    A slot is the request's row of the ReqToTokenPool.  Slots need no clearing: the kernels take the state as zero for a
+    sequence whose first row stands at position 0."""
+
+    def __init__(self, slots: int, width: int, taps: int, dtype: torch.dtype, device: str):
+        self.state = torch.zeros((slots, width), dtype=torch.float32, device=device)
+        self.conv = torch.zeros((slots, taps - 1, width), dtype=dtype, device=device)
+
+    def get_size_bytes(self):
+        return sum(t.numel() * t.element_size() for t in (self.state, self.conv))
+
+
+class HybridCache:
+    """What the layers of a decoder with mixed mixers keep between steps: one request table and one slot allocator for
+    all attention layers, a latent pool per attention layer and a state pool per recurrent layer (a layer that runs
+    several times has one of its own for every run).
+
+    layers: per layer run ("latent", latent, rotated part) or ("recurrent", width, taps).  The allocator's free list
+    lives on the host, where the engine lays its steps out."""
+
+    def __init__(self, layers, max_tokens: int, max_requests: int, max_context: int, dtype: torch.dtype, device):
+        self.req_pool = ReqToTokenPool(max_requests, max_context, device)
+        self.layers = []
+        for kind, a, b in layers:
+            if kind == "latent":
+                self.layers.append(MLATokenToKVPool(max_tokens, 1, dtype, a, b, 1, device))
+            else:
+                self.layers.append(RecurrentStatePool(max_requests, a, b, dtype, device))
+        self.allocator = TokenToKVPoolAllocator(max_tokens, dtype, "cpu", self)
+
+    def get_size_bytes(self):
+        return sum(p.get_kv_size_bytes() if isinstance(p, MLATokenToKVPool) else p.get_size_bytes() for p in self.layers)
