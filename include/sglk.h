@@ -1034,10 +1034,12 @@ SGLK_API int sglk_latent_rope_q(const void* src, int64_t src_m, int64_t src_h, v
                                 const float* cos_sin, const int32_t* positions, int M, int H, int rot_pitch, int rot_dims,
                                 int dtype, void* stream);
 /* out[m][h][n] = sum_k a[m][h][k] w[h][n][k].  bf16: w in operand order [H][Np / 16][K / 32][64 lanes][8] (lane 16 g + i:
- * column 16 s + i, k = 32 ks + 8 g + e); other types: row-major [H][Np][K].  lse != NULL: a holds the split partials
- * [M][H][splits][K] (fp32) of sglk_latent_decode, merged first. */
-SGLK_API int sglk_head_gemm(const void* a, const float* lse, int splits, int64_t a_m, int64_t a_h, const void* w, void* out,
-                            int M, int H, int N, int Np, int K, int64_t out_m, int64_t out_h, int dtype, void* stream);
+ * column 16 s + i, k = 32 ks + 8 g + e); other types: row-major [H][Np][K]. */
+SGLK_API int sglk_head_gemm(const void* a, int64_t a_m, int64_t a_h, const void* w, void* out, int M, int H, int N, int Np,
+                            int K, int64_t out_m, int64_t out_h, int dtype, void* stream);
+/* out[row][0 .. K) = merge of the split partials part [rows][splits][K] by their log-sum-exps lse [rows][splits] */
+SGLK_API int sglk_latent_merge(const float* part, const float* lse, int splits, void* out, int64_t rows, int K, int dtype,
+                               void* stream);
 SGLK_API int sglk_latent_decode_supported(int r_pitch, int rot_pitch);
 /* bf16 rows of one token each: q [M, H, r_pitch + rot_pitch] against the pool rows of positions (p - window, p] of request
  * req[m] (window <= 0: [0, p]); leaves `splits` normalised partials part [M][H][splits][r_pitch] and their

@@ -137,7 +137,8 @@ _SIGS = {
     "sglk_latent_prep": (i32, [p, i32, i32, i64, i64, p, p, p, i64, p, i64, p, p, p, i32, i32, i32, i32, i32,
         i32, i32, i32, f32, i32, p]),
     "sglk_latent_rope_q": (i32, [p, i64, i64, p, i64, i64, p, p, i32, i32, i32, i32, i32, p]),
-    "sglk_head_gemm": (i32, [p, p, i32, i64, i64, p, p, i32, i32, i32, i32, i32, i64, i64, i32, p]),
+    "sglk_head_gemm": (i32, [p, i64, i64, p, p, i32, i32, i32, i32, i32, i64, i64, i32, p]),
+    "sglk_latent_merge": (i32, [p, p, i32, p, i64, i32, i32, p]),
     "sglk_latent_decode_supported": (i32, [i32, i32]),
     "sglk_latent_decode": (i32, [p, i64, i64, p, i64, p, i64, p, p, p, p, i32, i32, i32, i32, i32, i32, f32,
         p]),

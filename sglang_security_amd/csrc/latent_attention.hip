@@ -19,7 +19,7 @@
 namespace sglk {
 
 // ---------------------------------------------------------------------------------------------------------------------
-// one block per token row
+// normalisation of both latents, rotation of the shared key part, pool write
 // ---------------------------------------------------------------------------------------------------------------------
 struct LatentPrep {
   RowSource src;           // columns [0, q_pitch) query latent, then r_pitch latent, then rot_dim rotated key part
@@ -36,56 +36,77 @@ struct LatentPrep {
   float eps;
 };
 
-template <typename T>
-__global__ void __launch_bounds__(256) latent_prep_kernel(LatentPrep a) {
-  extern __shared__ float rowbuf[];  // q_pitch + r_pitch + rot_pitch values
+// TPR threads per row (a wave, or the whole block), VPT pieces of eight elements per thread
+template <typename T, int TPR, int VPT>
+__global__ void __launch_bounds__(256) latent_prep_kernel(LatentPrep a, int M) {
+  extern __shared__ float rotbuf[];  // [256 / TPR][rot_pitch]
   __shared__ float red[2][4];
-  const int m = blockIdx.x;
-  const int cols = a.q_pitch + a.r_pitch + a.rot_pitch;
-  float sq = 0.f, sk = 0.f;
-  for (int v = threadIdx.x; v < cols / 8; v += 256) {
-    float t[8];
-    source8<T>(a.src, m, 8 * v, t);
+  const int t = threadIdx.x % TPR, sub = threadIdx.x / TPR;
+  const int m = blockIdx.x * (256 / TPR) + sub;
+  const bool row_ok = m < M;
+  const int row = row_ok ? m : M - 1;
+  const int vq = a.q_pitch / 8, vk = vq + a.r_pitch / 8, nv = vk + a.rot_pitch / 8;
+  float* rot = rotbuf + sub * a.rot_pitch;
+  float x[VPT][8], sq = 0.f, sk = 0.f;
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      rowbuf[8 * v + j] = t[j];
-      if (8 * v < a.q_pitch)
-        sq += t[j] * t[j];
-      else if (8 * v < a.q_pitch + a.r_pitch)
-        sk += t[j] * t[j];
+  for (int i = 0; i < VPT; ++i) {
+    const int v = t + TPR * i;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[i][j] = 0.f;
+    if (v >= nv) continue;
+    source8<T>(a.src, row, 8 * v, x[i]);
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) ss += x[i][j] * x[i][j];
+    if (v < vq)
+      sq += ss;
+    else if (v < vk)
+      sk += ss;
+    else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) rot[8 * (v - vk) + j] = x[i][j];
     }
   }
   sq = wave_sum(sq);
   sk = wave_sum(sk);
-  if ((threadIdx.x & 63) == 0) {
+  if (TPR > 64 && (threadIdx.x & 63) == 0) {
     red[0][threadIdx.x >> 6] = sq;
     red[1][threadIdx.x >> 6] = sk;
   }
   __syncthreads();
-  const float iq = 1.0f / sqrtf((red[0][0] + red[0][1] + red[0][2] + red[0][3]) / (float)a.q_rank + a.eps);
-  const float ik = 1.0f / sqrtf((red[1][0] + red[1][1] + red[1][2] + red[1][3]) / (float)a.kv_rank + a.eps);
-  for (int v = threadIdx.x; v < a.q_pitch / 8; v += 256) {
-    float t[8];
-#pragma unroll
-    for (int j = 0; j < 8; ++j) t[j] = rowbuf[8 * v + j] * iq * a.wq[8 * v + j];
-    st8<T>(a.cq, (int64_t)m * a.cq_stride + 8 * v, t);
+  if (TPR > 64) {
+    sq = red[0][0] + red[0][1] + red[0][2] + red[0][3];
+    sk = red[1][0] + red[1][1] + red[1][2] + red[1][3];
   }
+  if (!row_ok) return;
+  const float iq = 1.0f / sqrtf(sq / (float)a.q_rank + a.eps);
+  const float ik = 1.0f / sqrtf(sk / (float)a.kv_rank + a.eps);
   const int64_t slot = (int64_t)a.loc[m] * a.pool_stride;
-  for (int v = threadIdx.x; v < a.r_pitch / 8; v += 256) {
-    float t[8];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) t[j] = rowbuf[a.q_pitch + 8 * v + j] * ik * a.wkv[8 * v + j];
-    st8<T>(a.pool, slot + 8 * v, t);
+  for (int i = 0; i < VPT; ++i) {
+    const int v = t + TPR * i;
+    if (v >= vk) continue;
+    float w[8];
+    if (v < vq) {
+      ld8<float>(a.wq, 8 * v, w);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) w[j] *= x[i][j] * iq;
+      st8<T>(a.cq, (int64_t)m * a.cq_stride + 8 * v, w);
+    } else {
+      ld8<float>(a.wkv, 8 * (v - vq), w);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) w[j] *= x[i][j] * ik;
+      st8<T>(a.pool, slot + 8 * (v - vq), w);
+    }
   }
-  const float* kr = rowbuf + a.q_pitch + a.r_pitch;
   const float* cs = a.cos_sin + (int64_t)a.positions[m] * a.rot_dims;
   const int half = a.rot_dims / 2;
-  for (int d = threadIdx.x; d < a.rot_pitch; d += 256) {
-    float v = d < a.rot_dim ? kr[d] : 0.f;
+  for (int d = t; d < a.rot_pitch; d += TPR) {
+    float v = d < a.rot_dim ? rot[d] : 0.f;
     if (d < a.rot_dims) {
       const int i = d < half ? d : d - half;
       float ra, rb;
-      rope_pair(kr[i], kr[i + half], cs[i], cs[half + i], ra, rb);
+      rope_pair(rot[i], rot[i + half], cs[i], cs[half + i], ra, rb);
       v = d < half ? ra : rb;
     }
     st<T>(a.pool, slot + a.r_pitch + d, v);
@@ -117,97 +138,123 @@ __global__ void __launch_bounds__(256) latent_rope_q_kernel(const void* src, int
   st<T>(out, oi + i + half, rb);
 }
 
-// ---------------------------------------------------------------------------------------------------------------------
-// out[m][h][n] = sum_k a[m][h][k] * w[h][n][k].  Weights in operand order [H][Np / 16][K / 32][64 lanes][8]: every wave
-// streams its strips as consecutive memory; the 64 rows of a block sit in LDS.  MERGE: the rows are split partials of
-// an attention kernel ([M][H][S][K] fp32 + log-sum-exps [M][H][S]) that are merged on their way into LDS.
-// ---------------------------------------------------------------------------------------------------------------------
-constexpr int kHeadMaxK = 1024;
-constexpr int head_lds(int K) { return 64 * (K * 2 + 16); }
+// whole rows turned (rot_dims == rot_pitch), eight pairs per thread, rows 16-byte aligned
+template <typename T>
+__global__ void __launch_bounds__(256) latent_rope_q8_kernel(const void* src, int64_t src_m, int64_t src_h, void* out, int64_t out_m,
+                                                             int64_t out_h, const float* __restrict__ cos_sin,
+                                                             const int32_t* __restrict__ positions, int M, int H, int rot) {
+  const int half = rot / 2, per = half / 8;
+  const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (idx >= (int64_t)M * H * per) return;
+  const int i = (int)(idx % per) * 8;
+  const int mh = (int)(idx / per), h = mh % H, m = mh / H;
+  const int64_t si = m * src_m + h * src_h + i, oi = m * out_m + h * out_h + i;
+  const float* cs = cos_sin + (int64_t)positions[m] * rot + i;
+  float a[8], b[8], c[8], s[8];
+  ld8<T>(src, si, a);
+  ld8<T>(src, si + half, b);
+  ld8<float>(cs, 0, c);
+  ld8<float>(cs, half, s);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    float ra, rb;
+    rope_pair(a[j], b[j], c[j], s[j], ra, rb);
+    a[j] = ra;
+    b[j] = rb;
+  }
+  st8<T>(out, oi, a);
+  st8<T>(out, oi + half, b);
+}
 
-template <int NS, bool MERGE>
-__global__ void __launch_bounds__(256) head_gemm_kernel(const void* __restrict__ a, const float* __restrict__ lse, int S,
-                                                        int64_t a_m, int64_t a_h, const uint16_t* __restrict__ w,
-                                                        uint16_t* __restrict__ out, int M, int H, int N, int Np, int K,
-                                                        int64_t out_m, int64_t out_h) {
-  extern __shared__ __attribute__((aligned(16))) char lds[];
-  const int pitch = K * 2 + 16;
-  const int h = blockIdx.y, m0 = blockIdx.z * 64;
+// out[m][h][0 .. K) = the merged split partials part[m][h][S][K] (log-sum-exps lse [m][h][S]; -inf: nothing was left)
+template <typename T>
+__global__ void __launch_bounds__(256) latent_merge_kernel(const float* __restrict__ part, const float* __restrict__ lse, int S, int K,
+                                                           void* __restrict__ out, int64_t rows) {
+  const int nv = K / 8;
+  const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (idx >= rows * nv) return;
+  const int64_t row = idx / nv;
+  const int c = (int)(idx - row * nv) * 8;
+  const float* l = lse + row * S;
+  float e_max = -INFINITY;
+  for (int s = 0; s < S; ++s) e_max = fmaxf(e_max, l[s]);
+  float acc[8], tot = 0.f;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) acc[j] = 0.f;
+  for (int s0 = 0; s0 < S; s0 += 4) {  // four splits' loads in flight
+    float t[4][8], w[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      w[u] = s0 + u < S ? __expf(l[s0 + u] - e_max) : 0.f;
+      if (w[u] > 0.f) {
+        ld8<float>(part, (row * S + s0 + u) * K + c, t[u]);
+      } else {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) t[u][j] = 0.f;
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      tot += w[u];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) acc[j] = fmaf(w[u], t[u][j], acc[j]);
+    }
+  }
+  const float inv = 1.0f / tot;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) acc[j] *= inv;
+  st8<T>(out, row * K + c, acc);
+}
+
+// ---------------------------------------------------------------------------------------------------------------------
+// out[m][h][n] = sum_k a[m][h][k] * w[h][n][k].  Weights in operand order [H][Np / 16][K / 32][64 lanes][8].  Wave w of a
+// block owns rows 16 w .. of 64 and the block's NS strips of 16 columns; both operands go straight from memory into
+// registers, eight k-steps ahead (a head's product is too small to pay for a trip through LDS and its barrier).
+// ---------------------------------------------------------------------------------------------------------------------
+template <int NS>
+__global__ void __launch_bounds__(256) head_gemm_kernel(const uint16_t* __restrict__ a, int64_t a_m, int64_t a_h,
+                                                        const uint16_t* __restrict__ w, uint16_t* __restrict__ out, int M, int N,
+                                                        int Np, int K, int64_t out_m, int64_t out_h) {
+  const int h = blockIdx.y;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int i16 = lane & 15, g = lane >> 4;
-  const int ksteps = K / 32;
-  const int strip0 = (blockIdx.x * 4 + wid) * NS;
+  const int m0 = blockIdx.z * 64 + 16 * wid;
+  if (m0 >= M) return;
+  const int ksteps = K / 32, strip0 = blockIdx.x * NS;
+  const uint16_t* as = a + (int64_t)min(m0 + i16, M - 1) * a_m + h * a_h + 8 * g;  // rows past M repeat the last one
   const uint16_t* ws[NS];
 #pragma unroll
   for (int s = 0; s < NS; ++s)
     ws[s] = w + (((int64_t)h * (Np / 16) + min(strip0 + s, Np / 16 - 1)) * ksteps) * 512 + 8 * lane;
-  {
-    const int row = threadIdx.x >> 2, q = threadIdx.x & 3;
-    const int m = m0 + row;
-    const bool ok = m < M;
-    if constexpr (MERGE) {
-      float e_max = -INFINITY;
-      const float* l = lse + ((int64_t)min(m, M - 1) * H + h) * S;
-      for (int s = 0; s < S; ++s) e_max = fmaxf(e_max, l[s]);
-      float tot = 0.f;
-      for (int s = 0; s < S; ++s) tot += expf(l[s] - e_max);
-      const float inv = 1.0f / tot;
-      const float* base = reinterpret_cast<const float*>(a) + ((int64_t)min(m, M - 1) * H + h) * S * K;
-      for (int c = q; c < K / 8; c += 4) {
-        float acc[8];
+  float4v acc[NS];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) acc[j] = 0.f;
-        for (int s = 0; s < S; ++s) {
-          const float ls = l[s];
-          if (ls == -INFINITY) continue;  // an empty split left no partial
-          const float wt = expf(ls - e_max) * inv;
-          float t[8];
-          ld8<float>(base, (int64_t)s * K + 8 * c, t);
+  for (int s = 0; s < NS; ++s) acc[s] = float4v{0.f, 0.f, 0.f, 0.f};
+  constexpr int PF = 8;
+  for (int k0 = 0; k0 < ksteps; k0 += PF) {
+    short8 af[PF], bf[PF][NS];
 #pragma unroll
-          for (int j = 0; j < 8; ++j) acc[j] += wt * t[j];
-        }
-        if (!ok) {
+    for (int j = 0; j < PF; ++j) {
+      const int ks = min(k0 + j, ksteps - 1);
+      af[j] = *reinterpret_cast<const short8*>(as + 32 * ks);
 #pragma unroll
-          for (int j = 0; j < 8; ++j) acc[j] = 0.f;
-        }
-        st8<bf16_t>(lds + row * pitch, 8 * c, acc);
+      for (int s = 0; s < NS; ++s) bf[j][s] = *reinterpret_cast<const short8*>(ws[s] + 512 * ks);
+    }
+#pragma unroll
+    for (int j = 0; j < PF; ++j)
+      if (k0 + j < ksteps) {
+#pragma unroll
+        for (int s = 0; s < NS; ++s) acc[s] = Mfma16<bf16_t>::mma(af[j], bf[j][s], acc[s]);
       }
-    } else {
-      const uint16_t* src = reinterpret_cast<const uint16_t*>(a) + (int64_t)min(m, M - 1) * a_m + h * a_h;
-      for (int c = q; c < K / 8; c += 4)
-        *reinterpret_cast<int4v*>(lds + row * pitch + 16 * c) =
-            ok ? *reinterpret_cast<const int4v*>(src + 8 * c) : int4v{0, 0, 0, 0};
-    }
-  }
-  __syncthreads();
-  float4v acc[NS][4];
-#pragma unroll
-  for (int s = 0; s < NS; ++s)
-#pragma unroll
-    for (int mt = 0; mt < 4; ++mt) acc[s][mt] = float4v{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-  for (int ks = 0; ks < ksteps; ++ks) {
-    short8 b[NS];
-#pragma unroll
-    for (int s = 0; s < NS; ++s) b[s] = *reinterpret_cast<const short8*>(ws[s] + 512 * ks);
-#pragma unroll
-    for (int mt = 0; mt < 4; ++mt) {
-      const short8 af = *reinterpret_cast<const short8*>(lds + (16 * mt + i16) * pitch + (4 * ks + g) * 16);
-#pragma unroll
-      for (int s = 0; s < NS; ++s) acc[s][mt] = Mfma16<bf16_t>::mma(af, b[s], acc[s][mt]);
-    }
   }
 #pragma unroll
   for (int s = 0; s < NS; ++s) {
     const int n = (strip0 + s) * 16 + i16;
     if (n >= N) continue;
 #pragma unroll
-    for (int mt = 0; mt < 4; ++mt)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int m = m0 + 16 * mt + 4 * g + r;
-        if (m < M) out[m * out_m + h * out_h + n] = Conv<bf16_t>::from_f32(acc[s][mt][r]);
-      }
+    for (int r = 0; r < 4; ++r) {
+      const int m = m0 + 4 * g + r;
+      if (m < M) out[m * out_m + h * out_h + n] = Conv<bf16_t>::from_f32(acc[s][r]);
+    }
   }
 }
 
@@ -521,11 +568,28 @@ int sglk_latent_prep(const void* src, int src_f32, int splits, int64_t part_stri
   SGLK_CHECK(src && wq && wkv && cq && pool && loc && cos_sin && positions, "latent_prep: null pointer");
   SGLK_CHECK(aligned16(cq) && aligned16(pool), "latent_prep: rows must be 16-byte aligned");
   const int cols = q_pitch + r_pitch + rot_pitch;
-  SGLK_CHECK(cols <= 12288, "latent_prep: rows of at most 12288 elements");
+  SGLK_CHECK(cols <= 16384 && rot_pitch <= 1024, "latent_prep: rows of at most 16384 elements, 1024 of them rotated");
+  SGLK_CHECK(aligned16(wq) && aligned16(wkv), "latent_prep: norm weights must be 16-byte aligned");
   if (int rc = check_source(src, src_f32, splits, part_stride, src_stride, cols, dtype, "latent_prep")) return rc;
   LatentPrep a{RowSource{src, src_f32, splits, part_stride, src_stride}, wq, wkv, cq, cq_stride, pool, pool_stride, loc, cos_sin,
                positions, q_rank, q_pitch, kv_rank, r_pitch, rot_dim, rot_pitch, rot_dims, eps};
-  SGLK_DISPATCH_FLOAT(dtype, T, hipLaunchKernelGGL((latent_prep_kernel<T>), dim3(M), dim3(256), cols * 4, (hipStream_t)stream, a));
+  // many rows: a wave each; a decode batch: a block each
+  const bool waves = M > 512 && cols <= 64 * 8 * 8;
+  const int vpt = (cols / 8 + (waves ? 63 : 255)) / (waves ? 64 : 256);
+#define SGLK_PREP(TPR, V)                                                                                                     \
+  hipLaunchKernelGGL((latent_prep_kernel<T, TPR, V>), dim3((M + 256 / TPR - 1) / (256 / TPR)), dim3(256),                     \
+                     (256 / TPR) * rot_pitch * 4, (hipStream_t)stream, a, M)
+  SGLK_DISPATCH_FLOAT(dtype, T, {
+    if (waves && vpt <= 5)
+      SGLK_PREP(64, 5);
+    else if (waves)
+      SGLK_PREP(64, 8);
+    else if (vpt <= 2)
+      SGLK_PREP(256, 2);
+    else
+      SGLK_PREP(256, 8);
+  });
+#undef SGLK_PREP
   SGLK_LAUNCH_CHECK();
   return SGLK_OK;
 }
@@ -538,6 +602,17 @@ int sglk_latent_rope_q(const void* src, int64_t src_m, int64_t src_h, void* out,
   SGLK_CHECK(src_h >= rot_pitch && out_h >= rot_pitch, "latent_rope_q: head stride too small");
   if (M == 0) return SGLK_OK;
   SGLK_CHECK(src && out && cos_sin && positions, "latent_rope_q: null pointer");
+  const bool wide = rot_dims == rot_pitch && rot_dims % 16 == 0 && aligned16(src) && aligned16(out) && aligned16(cos_sin) &&
+                    src_m % 8 == 0 && src_h % 8 == 0 && out_m % 8 == 0 && out_h % 8 == 0 && (int64_t)M * H < (1 << 30);
+  if (wide) {
+    const int64_t threads = (int64_t)M * H * (rot_dims / 16);
+    SGLK_DISPATCH_FLOAT(dtype, T,
+                        hipLaunchKernelGGL((latent_rope_q8_kernel<T>), dim3((unsigned)((threads + 255) / 256)), dim3(256), 0,
+                                           (hipStream_t)stream, src, src_m, src_h, out, out_m, out_h, cos_sin, positions, M, H,
+                                           rot_dims));
+    SGLK_LAUNCH_CHECK();
+    return SGLK_OK;
+  }
   const int64_t total = (int64_t)M * H * (rot_pitch - rot_dims / 2);
   SGLK_DISPATCH_FLOAT(dtype, T,
                       hipLaunchKernelGGL((latent_rope_q_kernel<T>), dim3((unsigned)((total + 255) / 256)), dim3(256), 0,
@@ -547,14 +622,13 @@ int sglk_latent_rope_q(const void* src, int64_t src_m, int64_t src_h, void* out,
   return SGLK_OK;
 }
 
-int sglk_head_gemm(const void* a, const float* lse, int splits, int64_t a_m, int64_t a_h, const void* w, void* out, int M, int H,
-                   int N, int Np, int K, int64_t out_m, int64_t out_h, int dtype, void* stream) {
+int sglk_head_gemm(const void* a, int64_t a_m, int64_t a_h, const void* w, void* out, int M, int H, int N, int Np, int K,
+                   int64_t out_m, int64_t out_h, int dtype, void* stream) {
   SGLK_CHECK(M >= 0 && H > 0 && N > 0 && Np >= N && Np % 16 == 0 && K > 0 && K % 32 == 0, "head_gemm: bad shape");
   if (M == 0) return SGLK_OK;
   SGLK_CHECK(a && w && out, "head_gemm: null pointer");
-  SGLK_CHECK(out_h >= N && (lse || a_h >= K), "head_gemm: head stride too small");
+  SGLK_CHECK(out_h >= N && a_h >= K, "head_gemm: head stride too small");
   if (dtype != SGLK_BF16) {
-    SGLK_CHECK(!lse, "head_gemm: split partials are merged for bf16 only");
     const int64_t total = (int64_t)M * H * N;
     SGLK_DISPATCH_FLOAT(dtype, T,
                         hipLaunchKernelGGL((head_gemm_rows_kernel<T>), dim3((unsigned)((total + 255) / 256)), dim3(256), 0,
@@ -562,29 +636,29 @@ int sglk_head_gemm(const void* a, const float* lse, int splits, int64_t a_m, int
     SGLK_LAUNCH_CHECK();
     return SGLK_OK;
   }
-  SGLK_CHECK(K <= kHeadMaxK, "head_gemm: K=%d, at most %d", K, kHeadMaxK);
-  SGLK_CHECK(aligned16(a) && aligned16(w) && (lse || (a_m % 8 == 0 && a_h % 8 == 0)), "head_gemm: rows must be 16-byte aligned");
-  SGLK_CHECK(!lse || splits >= 1, "head_gemm: bad split count");
-  const int ns = Np > 64 ? 2 : 1;
-  const dim3 grid((Np / 16 + 4 * ns - 1) / (4 * ns), H, (M + 63) / 64);
-#define SGLK_HG(NS, MG)                                                                                                   \
-  do {                                                                                                                    \
-    if (int rc = ensure_lds<head_gemm_kernel<NS, MG>>(head_lds(kHeadMaxK))) return rc;                                    \
-    hipLaunchKernelGGL((head_gemm_kernel<NS, MG>), grid, dim3(256), head_lds(K), (hipStream_t)stream, a, lse, splits, a_m, a_h, \
-                       (const uint16_t*)w, (uint16_t*)out, M, H, N, Np, K, out_m, out_h);                                 \
-  } while (0)
-  if (lse) {
-    if (ns == 2)
-      SGLK_HG(2, true);
-    else
-      SGLK_HG(1, true);
-  } else {
-    if (ns == 2)
-      SGLK_HG(2, false);
-    else
-      SGLK_HG(1, false);
-  }
+  SGLK_CHECK(aligned16(a) && aligned16(w) && a_m % 8 == 0 && a_h % 8 == 0, "head_gemm: rows must be 16-byte aligned");
+  const int ns = (int64_t)H * (Np / 32) >= 256 ? 2 : 1;  // two strips per wave where that still covers the chip
+  const dim3 grid((Np / 16 + ns - 1) / ns, H, (M + 63) / 64);
+#define SGLK_HG(NS)                                                                                                       \
+  hipLaunchKernelGGL((head_gemm_kernel<NS>), grid, dim3(256), 0, (hipStream_t)stream, (const uint16_t*)a, a_m, a_h,       \
+                     (const uint16_t*)w, (uint16_t*)out, M, N, Np, K, out_m, out_h)
+  if (ns == 2)
+    SGLK_HG(2);
+  else
+    SGLK_HG(1);
 #undef SGLK_HG
+  SGLK_LAUNCH_CHECK();
+  return SGLK_OK;
+}
+
+int sglk_latent_merge(const float* part, const float* lse, int splits, void* out, int64_t rows, int K, int dtype, void* stream) {
+  SGLK_CHECK(rows >= 0 && splits >= 1 && K > 0 && K % 8 == 0, "latent_merge: bad shape");
+  if (rows == 0) return SGLK_OK;
+  SGLK_CHECK(part && lse && out && aligned16(part) && aligned16(out), "latent_merge: null or unaligned pointer");
+  const int64_t vecs = rows * (K / 8);
+  SGLK_DISPATCH_FLOAT(dtype, T,
+                      hipLaunchKernelGGL((latent_merge_kernel<T>), dim3((unsigned)((vecs + 255) / 256)), dim3(256), 0,
+                                         (hipStream_t)stream, part, lse, splits, K, out, rows));
   SGLK_LAUNCH_CHECK();
   return SGLK_OK;
 }

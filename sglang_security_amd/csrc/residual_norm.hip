@@ -153,9 +153,17 @@ __global__ void __launch_bounds__(256) capped_logits_kernel(RowSource src, float
   const int m = (int)(idx / nv), n = (int)(idx - (int64_t)m * nv) * 8;
   float v[8];
   source8<T>(src, m, n, v);
+  if (cap > 0.f) {
 #pragma unroll
-  for (int j = 0; j < 8; ++j)
-    if (n + j < V) out[(int64_t)m * out_stride + n + j] = cap > 0.f ? cap * tanhf(v[j] / cap) : v[j];
+    for (int j = 0; j < 8; ++j) v[j] = cap * tanhf(v[j] / cap);
+  }
+  if (n + 8 <= V && (out_stride & 3) == 0) {
+    st8<float>(out, (int64_t)m * out_stride + n, v);
+  } else {
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      if (n + j < V) out[(int64_t)m * out_stride + n + j] = v[j];
+  }
 }
 
 // req_to_token[req[seq[t]]][pos[t]] = loc[t]
@@ -229,7 +237,7 @@ int sglk_capped_logits(const void* src, int src_f32, int splits, int64_t part_st
                        int N, int V, int64_t out_stride, float cap, int dtype, void* stream) {
   SGLK_CHECK(M >= 0 && V > 0 && N >= V && N % 8 == 0 && out_stride >= V, "capped_logits: bad shape");
   if (M == 0) return SGLK_OK;
-  SGLK_CHECK(src && out, "capped_logits: null pointer");
+  SGLK_CHECK(src && out && aligned16(out), "capped_logits: null or unaligned pointer");
   if (int rc = check_source(src, src_f32, splits, part_stride, src_stride, N, dtype, "capped_logits")) return rc;
   const int64_t vecs = (int64_t)M * (N / 8);
   SGLK_DISPATCH_FLOAT(dtype, T,

@@ -50,6 +50,19 @@ __device__ __forceinline__ void gate_terms(float zr, float zi, float sp, float u
   b = sqrtf(fmaxf(-expm1f(2.0f * la), 0.f)) * sigmoidf(zi) * u;
 }
 
+// The tile kernels' form on the hardware exponential (base 2) and reciprocal.  zr, zi: products without their biases; nbr, nbi:
+// biases * -log2(e); sp8: softplus(lambda) * -8 log2(e).  1 - a^2 by its series where it is small.
+constexpr float kLog2e = 1.4426950408889634f;
+__device__ __forceinline__ void gate_terms_fast(float zr, float zi, float nbr, float nbi, float sp8, float u, float& a, float& b) {
+  const float sr = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(fmaf(zr, -kLog2e, nbr)));
+  const float si = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(fmaf(zi, -kLog2e, nbi)));
+  const float la = sr * sp8;  // log2 of the decay
+  a = __builtin_amdgcn_exp2f(la);
+  const float x = la * (2.0f / kLog2e);
+  const float near = -x * fmaf(x, fmaf(x, fmaf(x, 0.041666667f, 0.16666667f), 0.5f), 1.0f);
+  b = __builtin_amdgcn_sqrtf(x > -0.03f ? near : fmaf(-a, a, 1.0f)) * si * u;
+}
+
 struct RglruConv {
   RowSource src;          // columns [0, W) x branch, [W, 2 W) y branch
   const float* bx;        // [W]
@@ -71,53 +84,87 @@ __device__ __forceinline__ void conv_input8(const RglruConv& a, int m, int c, co
   for (int j = 0; j < 8; ++j) x[j] = round_to<T>(x[j] + bias[j]);
 }
 
-template <typename T>
+// One thread: eight channels of R rows; blockIdx.y 0: the x branch, 1: the y branch.
+template <typename T, int R>
 __global__ void __launch_bounds__(256) rglru_conv_kernel(RglruConv a) {
   const int nv = a.W / 8;
   const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
-  if (idx >= (int64_t)a.M * nv) return;
-  const int m = (int)(idx / nv), c = (int)(idx - (int64_t)m * nv) * 8;
-  float t[8], acc[8];
-  ld8<float>(a.by, c, t);
-  source8<T>(a.src, m, a.W + c, acc);
+  if (idx >= (int64_t)((a.M + R - 1) / R) * nv) return;
+  const int m0 = (int)(idx / nv) * R, c = (int)(idx % nv) * 8;
+  float bias[8], acc[8];
+  if (blockIdx.y) {
+    ld8<float>(a.by, c, bias);
 #pragma unroll
-  for (int j = 0; j < 8; ++j) acc[j] = gelu_tanh(acc[j] + t[j]);
-  st8<T>(a.y, (int64_t)m * a.W + c, acc);
-
-  const int s = a.seq.row_seq[m];
-  const int start = a.seq.start[s];
-  const int k = m - a.seq.row0[s];  // row within its sequence's portion
-  const int keep = a.taps - 1;
-  const int64_t st0 = (int64_t)a.seq.slot[s] * keep * a.W + c;
-  float bias[8], x[8], w[8];
-  ld8<float>(a.bx, c, bias);
-  ld8<float>(a.conv_b, c, acc);
-  for (int d = keep; d >= 0; --d) {  // d rows back
-    if (k - d >= 0) {
-      conv_input8<T>(a, m - d, c, bias, x);
-    } else if (start > 0) {
-      ld8<T>(a.state, st0 + (int64_t)(keep + k - d) * a.W, x);
-    } else {
-      continue;
+    for (int r = 0; r < R; ++r) {
+      const int m = m0 + r;
+      if (m >= a.M) break;
+      source8<T>(a.src, m, a.W + c, acc);
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        acc[j] = sizeof(typename Raw<T>::type) == 4 ? gelu_tanh(acc[j] + bias[j]) : gelu_tanh_fast(acc[j] + bias[j]);
+      st8<T>(a.y, (int64_t)m * a.W + c, acc);
     }
-    ld8<float>(a.conv, (int64_t)(keep - d) * a.W + c, w);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) acc[j] = fmaf(x[j], w[j], acc[j]);
+    return;
   }
-  st8<T>(a.u, (int64_t)m * a.W + c, acc);
-  if (m < a.singles && keep > 0) {
-    // x holds the row's own input: shift the state by one
-    float o[8];
-    for (int j = 0; j + 1 < keep; ++j) {
-      if (start > 0) {
-        ld8<T>(a.state, st0 + (int64_t)(j + 1) * a.W, o);
-      } else {
+  ld8<float>(a.bx, c, bias);
+  const int keep = a.taps - 1;
+  if constexpr (R > 1) {
+    // four taps, rows of one sequence with everything they need in this step: every input is formed once
+    const int s = a.seq.row_seq[m0];
+    if (keep == 3 && m0 + R <= a.M && a.seq.row_seq[m0 + R - 1] == s && m0 - a.seq.row0[s] >= 3) {
+      float x[R + 3][8], w[4][8], cb[8];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) o[e] = 0.f;
+      for (int r = 0; r < R + 3; ++r) conv_input8<T>(a, m0 - 3 + r, c, bias, x[r]);
+#pragma unroll
+      for (int t = 0; t < 4; ++t) ld8<float>(a.conv, (int64_t)t * a.W + c, w[t]);
+      ld8<float>(a.conv_b, c, cb);
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          acc[j] = cb[j];
+#pragma unroll
+          for (int t = 0; t < 4; ++t) acc[j] = fmaf(x[r + t][j], w[t][j], acc[j]);
+        }
+        st8<T>(a.u, (int64_t)(m0 + r) * a.W + c, acc);
       }
-      st8<T>(a.state, st0 + (int64_t)j * a.W, o);
+      return;
     }
-    st8<T>(a.state, st0 + (int64_t)(keep - 1) * a.W, x);
+  }
+  for (int m = m0; m < min(m0 + R, a.M); ++m) {
+    const int s = a.seq.row_seq[m];
+    const int start = a.seq.start[s];
+    const int k = m - a.seq.row0[s];  // row within its sequence's portion
+    const int64_t st0 = (int64_t)a.seq.slot[s] * keep * a.W + c;
+    float x[8], w[8];
+    ld8<float>(a.conv_b, c, acc);
+    for (int d = keep; d >= 0; --d) {  // d rows back
+      if (k - d >= 0) {
+        conv_input8<T>(a, m - d, c, bias, x);
+      } else if (start > 0) {
+        ld8<T>(a.state, st0 + (int64_t)(keep + k - d) * a.W, x);
+      } else {
+        continue;
+      }
+      ld8<float>(a.conv, (int64_t)(keep - d) * a.W + c, w);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) acc[j] = fmaf(x[j], w[j], acc[j]);
+    }
+    st8<T>(a.u, (int64_t)m * a.W + c, acc);
+    if (m < a.singles && keep > 0) {
+      // x holds the row's own input: shift the state by one
+      float o[8];
+      for (int j = 0; j + 1 < keep; ++j) {
+        if (start > 0) {
+          ld8<T>(a.state, st0 + (int64_t)(j + 1) * a.W, o);
+        } else {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) o[e] = 0.f;
+        }
+        st8<T>(a.state, st0 + (int64_t)j * a.W, o);
+      }
+      st8<T>(a.state, st0 + (int64_t)(keep - 1) * a.W, x);
+    }
   }
 }
 
@@ -169,29 +216,109 @@ __global__ void __launch_bounds__(256) rglru_step_kernel(RglruGates a, const uin
   const int ksteps = a.bwp / 32, pitch = a.bwp * 2 + 16;
   const int64_t wo = (((int64_t)b * (a.bwp / 16) + strip) * ksteps) * 512 + 8 * lane;
   const int c = b * a.bwp + 16 * strip + i16;
+  // eight k-steps of both weights, the state and the gate vectors are on their way before the rows are parked
+  constexpr int PF = 8;
+  short8 wr[PF], wi[PF];
+  auto fetch = [&](int k0) {
+#pragma unroll
+    for (int j = 0; j < PF; ++j)
+      if (k0 + j < ksteps) {
+        wr[j] = *reinterpret_cast<const short8*>(a.wr + wo + 512 * (k0 + j));
+        wi[j] = *reinterpret_cast<const short8*>(a.wi + wo + 512 * (k0 + j));
+      }
+  };
+  fetch(0);
+  const float br = a.br[c] * -kLog2e, bi = a.bi[c] * -kLog2e, sp = a.sp[c] * (-8.0f * kLog2e);
+  float old[4], yv[4];
+  float* sl[4];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int m = min(m0 + 16 * wid + 4 * g + r, a.M - 1);
+    sl[r] = state + (int64_t)slot[m] * a.W + c;
+    old[r] = start[m] > 0 ? *sl[r] : 0.f;
+    yv[r] = Conv<bf16_t>::to_f32(y[(int64_t)m * a.W + c]);
+  }
   park_u(lds, a.u, a.W, m0, min(64, a.M - m0), b * a.bwp, a.bwp);
   __syncthreads();
   if (m0 + 16 * wid >= a.M) return;
   float4v ar = float4v{0.f, 0.f, 0.f, 0.f}, ai = ar;
-  for (int ks = 0; ks < ksteps; ++ks) {
-    const short8 wr = *reinterpret_cast<const short8*>(a.wr + wo + 512 * ks);
-    const short8 wi = *reinterpret_cast<const short8*>(a.wi + wo + 512 * ks);
-    const short8 af = *reinterpret_cast<const short8*>(lds + (16 * wid + i16) * pitch + (4 * ks + g) * 16);
-    ar = Mfma16<bf16_t>::mma(af, wr, ar);
-    ai = Mfma16<bf16_t>::mma(af, wi, ai);
+  for (int k0 = 0; k0 < ksteps; k0 += PF) {
+    if (k0 > 0) fetch(k0);
+#pragma unroll
+    for (int j = 0; j < PF; ++j)
+      if (k0 + j < ksteps) {
+        const short8 af = *reinterpret_cast<const short8*>(lds + (16 * wid + i16) * pitch + (4 * (k0 + j) + g) * 16);
+        ar = Mfma16<bf16_t>::mma(af, wr[j], ar);
+        ai = Mfma16<bf16_t>::mma(af, wi[j], ai);
+      }
   }
-  const float br = a.br[c], bi = a.bi[c], sp = a.sp[c];
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int m = m0 + 16 * wid + 4 * g + r;
     if (m >= a.M) continue;
     const float u = Conv<bf16_t>::to_f32(*reinterpret_cast<const uint16_t*>(lds + (m - m0) * pitch + (16 * strip + i16) * 2));
     float da, db;
-    gate_terms(ar[r] + br, ai[r] + bi, sp, u, da, db);
-    float* sl = state + (int64_t)slot[m] * a.W + c;
-    const float S = (start[m] > 0 ? da * *sl : 0.f) + db;
-    *sl = S;
-    out[(int64_t)m * out_stride + c] = Conv<bf16_t>::from_f32(S * Conv<bf16_t>::to_f32(y[(int64_t)m * a.W + c]));
+    gate_terms_fast(ar[r], ai[r], br, bi, sp, u, da, db);
+    const float S = fmaf(da, old[r], db);
+    *sl[r] = S;
+    out[(int64_t)m * out_stride + c] = Conv<bf16_t>::from_f32(S * yv[r]);
+  }
+}
+
+// The recurrence over the 64 rows of a tile, one channel per lane group: lane (i16, g) holds rows 16 mt + 4 g + r of its
+// channel, so it runs over r inside the lane, over g with two shuffles, over mt in sequence.  ucol: the channel's column of
+// the u rows in LDS; h, p: the tile's first row of the outputs.
+template <bool FULL>
+__device__ __forceinline__ void tile_scan(const float4v (&ar)[4], const float4v (&ai)[4], float br, float bi, float sp,
+                                          const char* ucol, int pitch, int valid, int W, int c, float* __restrict__ h,
+                                          float* __restrict__ p) {
+  const int lane = threadIdx.x & 63, i16 = lane & 15, g = lane >> 4;
+  const uint32_t off = (uint32_t)(4 * g) * W + c;
+  float P0 = 1.f, H0 = 0.f;  // decay product and state over the rows in front
+#pragma unroll
+  for (int mt = 0; mt < 4; ++mt) {
+    float A[4], B[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int k = 16 * mt + 4 * g + r;
+      const float u = Conv<bf16_t>::to_f32(*reinterpret_cast<const uint16_t*>(ucol + k * pitch));
+      gate_terms_fast(ar[mt][r], ai[mt][r], br, bi, sp, u, A[r], B[r]);
+      if (!FULL && k >= valid) {
+        A[r] = 1.f;
+        B[r] = 0.f;
+      }
+      if (r > 0) {
+        B[r] = fmaf(A[r], B[r - 1], B[r]);
+        A[r] *= A[r - 1];
+      }
+    }
+    // inclusive scan of (A[3], B[3]) over g, then the exclusive one
+    float sa = A[3], sb = B[3];
+#pragma unroll
+    for (int o = 16; o < 64; o <<= 1) {
+      const float pa = __shfl_up(sa, o, 64), pb = __shfl_up(sb, o, 64);
+      if (lane >= o) {
+        sb = fmaf(sa, pb, sb);
+        sa *= pa;
+      }
+    }
+    float ea = __shfl_up(sa, 16, 64), eb = __shfl_up(sb, 16, 64);
+    if (lane < 16) {
+      ea = 1.f;
+      eb = 0.f;
+    }
+    const float pin = ea * P0, hin = fmaf(ea, H0, eb);  // everything in front of this lane's four rows
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const uint32_t o = (uint32_t)(16 * mt + r) * W + off;
+      if (FULL || 16 * mt + 4 * g + r < valid) {
+        h[o] = fmaf(A[r], hin, B[r]);
+        p[o] = A[r] * pin;
+      }
+    }
+    const float ta = __shfl(sa, 48 + i16, 64), tb = __shfl(sb, 48 + i16, 64);
+    H0 = fmaf(ta, H0, tb);
+    P0 *= ta;
   }
 }
 
@@ -200,78 +327,46 @@ __global__ void __launch_bounds__(256) rglru_gates_kernel(RglruGates a, const in
                                                           const int32_t* __restrict__ tile_rows, float* __restrict__ hloc,
                                                           float* __restrict__ prod) {
   extern __shared__ __attribute__((aligned(16))) char lds[];
-  const int row0 = tile_row[blockIdx.x], valid = tile_rows[blockIdx.x], b = blockIdx.y;
+  // channel blocks run fastest: the blocks in flight then write whole rows, not one column strip of many rows
+  const int row0 = tile_row[blockIdx.y], valid = tile_rows[blockIdx.y], b = blockIdx.x;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int i16 = lane & 15, g = lane >> 4;
   const int ksteps = a.bwp / 32, strips = a.bwp / 16, pitch = a.bwp * 2 + 16;
   park_u(lds, a.u, a.W, row0, valid, b * a.bwp, a.bwp);
   __syncthreads();
+  constexpr int PF = 8;
   for (int strip = wid + 4 * blockIdx.z; strip < strips; strip += 4 * gridDim.z) {
     const int64_t wo = (((int64_t)b * strips + strip) * ksteps) * 512 + 8 * lane;
     const int c = b * a.bwp + 16 * strip + i16;
     float4v ar[4], ai[4];
 #pragma unroll
     for (int mt = 0; mt < 4; ++mt) ar[mt] = ai[mt] = float4v{0.f, 0.f, 0.f, 0.f};
-    for (int ks = 0; ks < ksteps; ++ks) {
-      const short8 wr = *reinterpret_cast<const short8*>(a.wr + wo + 512 * ks);
-      const short8 wi = *reinterpret_cast<const short8*>(a.wi + wo + 512 * ks);
+    for (int k0 = 0; k0 < ksteps; k0 += PF) {
+      short8 wr[PF], wi[PF];  // a strip's weights come from L2: eight k-steps in flight
 #pragma unroll
-      for (int mt = 0; mt < 4; ++mt) {
-        const short8 af = *reinterpret_cast<const short8*>(lds + (16 * mt + i16) * pitch + (4 * ks + g) * 16);
-        ar[mt] = Mfma16<bf16_t>::mma(af, wr, ar[mt]);
-        ai[mt] = Mfma16<bf16_t>::mma(af, wi, ai[mt]);
+      for (int j = 0; j < PF; ++j) {
+        const int ks = min(k0 + j, ksteps - 1);
+        wr[j] = *reinterpret_cast<const short8*>(a.wr + wo + 512 * ks);
+        wi[j] = *reinterpret_cast<const short8*>(a.wi + wo + 512 * ks);
+      }
+#pragma unroll
+      for (int j = 0; j < PF; ++j) {
+        if (k0 + j >= ksteps) break;
+#pragma unroll
+        for (int mt = 0; mt < 4; ++mt) {
+          const short8 af = *reinterpret_cast<const short8*>(lds + (16 * mt + i16) * pitch + (4 * (k0 + j) + g) * 16);
+          ar[mt] = Mfma16<bf16_t>::mma(af, wr[j], ar[mt]);
+          ai[mt] = Mfma16<bf16_t>::mma(af, wi[j], ai[mt]);
+        }
       }
     }
-    const float br = a.br[c], bi = a.bi[c], sp = a.sp[c];
-    // Lane (i16, g) holds rows 16 mt + 4 g + r of its channel: the recurrence runs over r inside the lane, over g with
-    // two shuffles, over mt in sequence.
-    float P0 = 1.f, H0 = 0.f;  // decay product and state over the rows in front
-#pragma unroll
-    for (int mt = 0; mt < 4; ++mt) {
-      float A[4], B[4];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int k = 16 * mt + 4 * g + r;
-        const float u = Conv<bf16_t>::to_f32(*reinterpret_cast<const uint16_t*>(lds + k * pitch + (16 * strip + i16) * 2));
-        gate_terms(ar[mt][r] + br, ai[mt][r] + bi, sp, u, A[r], B[r]);
-        if (k >= valid) {
-          A[r] = 1.f;
-          B[r] = 0.f;
-        }
-        if (r > 0) {
-          B[r] = fmaf(A[r], B[r - 1], B[r]);
-          A[r] *= A[r - 1];
-        }
-      }
-      // inclusive scan of (A[3], B[3]) over g, then the exclusive one
-      float sa = A[3], sb = B[3];
-#pragma unroll
-      for (int o = 16; o < 64; o <<= 1) {
-        const float pa = __shfl_up(sa, o, 64), pb = __shfl_up(sb, o, 64);
-        if (lane >= o) {
-          sb = fmaf(sa, pb, sb);
-          sa *= pa;
-        }
-      }
-      float ea = __shfl_up(sa, 16, 64), eb = __shfl_up(sb, 16, 64);
-      if (lane < 16) {
-        ea = 1.f;
-        eb = 0.f;
-      }
-      const float pin = ea * P0, hin = fmaf(ea, H0, eb);  // everything in front of this lane's four rows
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int k = 16 * mt + 4 * g + r;
-        if (k < valid) {
-          const int64_t o = (int64_t)(row0 + k) * a.W + c;
-          hloc[o] = fmaf(A[r], hin, B[r]);
-          prod[o] = A[r] * pin;
-        }
-      }
-      const float ta = __shfl(sa, 48 + i16, 64), tb = __shfl(sb, 48 + i16, 64);
-      H0 = fmaf(ta, H0, tb);
-      P0 *= ta;
-    }
+    const float br = a.br[c] * -kLog2e, bi = a.bi[c] * -kLog2e, sp = a.sp[c] * (-8.0f * kLog2e);
+    if (valid == kScanTile)
+      tile_scan<true>(ar, ai, br, bi, sp, lds + (16 * strip + i16) * 2, pitch, valid, a.W, c, hloc + (int64_t)row0 * a.W,
+                      prod + (int64_t)row0 * a.W);
+    else
+      tile_scan<false>(ar, ai, br, bi, sp, lds + (16 * strip + i16) * 2, pitch, valid, a.W, c, hloc + (int64_t)row0 * a.W,
+                       prod + (int64_t)row0 * a.W);
   }
 }
 
@@ -401,10 +496,15 @@ int sglk_rglru_conv(SGLK_CONV_ARGS, int dtype, void* stream) {
   SGLK_CONV_MAKE;
   if (int rc = check_conv(a, src_f32, splits, part_stride, src_stride, n_seqs, dtype, "rglru_conv")) return rc;
   if (M == 0) return SGLK_OK;
-  const int64_t vecs = (int64_t)M * (W / 8);
-  SGLK_DISPATCH_FLOAT(dtype, T,
-                      hipLaunchKernelGGL((rglru_conv_kernel<T>), dim3((unsigned)((vecs + 255) / 256)), dim3(256), 0,
-                                         (hipStream_t)stream, a));
+  const int per = M >= 256 ? 4 : 1;  // rows per thread
+  const int64_t threads = (int64_t)((M + per - 1) / per) * (W / 8);
+  const dim3 grid((unsigned)((threads + 255) / 256), 2);
+  SGLK_DISPATCH_FLOAT(dtype, T, {
+    if (per == 4)
+      hipLaunchKernelGGL((rglru_conv_kernel<T, 4>), grid, dim3(256), 0, (hipStream_t)stream, a);
+    else
+      hipLaunchKernelGGL((rglru_conv_kernel<T, 1>), grid, dim3(256), 0, (hipStream_t)stream, a);
+  });
   SGLK_LAUNCH_CHECK();
   return SGLK_OK;
 }
@@ -436,7 +536,7 @@ int sglk_rglru_step(const void* u, const void* wr, const void* wi, const float* 
 int sglk_rglru_gates(const void* u, const void* wr, const void* wi, const float* br, const float* bi, const float* sp,
                      const int32_t* tile_row, const int32_t* tile_rows, int tiles, float* hloc, float* prod, int W, int bwp,
                      int blocks, void* stream) {
-  SGLK_CHECK(tiles >= 0, "rglru_gates: bad shape");
+  SGLK_CHECK(tiles >= 0 && tiles <= 65535, "rglru_gates: at most 65535 tiles");
   if (tiles == 0) return SGLK_OK;
   if (int rc = check_gates(u, wr, wi, br, bi, sp, W, bwp, blocks, "rglru_gates")) return rc;
   SGLK_CHECK(tile_row && tile_rows && hloc && prod, "rglru_gates: null pointer");
@@ -445,7 +545,7 @@ int sglk_rglru_gates(const void* u, const void* wr, const void* wi, const float*
   // a few tiles only: the strips of a channel block spread over more blocks
   const int groups = (bwp / 16 + 3) / 4;
   const int z = std::max(1, std::min(groups, 1024 / std::max(tiles * blocks, 1)));
-  hipLaunchKernelGGL(rglru_gates_kernel, dim3(tiles, blocks, z), dim3(256), gate_lds(bwp), (hipStream_t)stream, a, tile_row,
+  hipLaunchKernelGGL(rglru_gates_kernel, dim3(blocks, tiles, z), dim3(256), gate_lds(bwp), (hipStream_t)stream, a, tile_row,
                      tile_rows, hloc, prod);
   SGLK_LAUNCH_CHECK();
   return SGLK_OK;

@@ -71,6 +71,12 @@ __device__ __forceinline__ float gelu_tanh(float z) {
   return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 
+// the same through the hardware exponential and reciprocal, for results that are rounded to 16 bits
+__device__ __forceinline__ float gelu_tanh_fast(float z) {
+  const float t = 0.7978845608028654f * (z + 0.044715f * z * z * z);
+  return z * (1.0f - __builtin_amdgcn_rcpf(1.0f + __expf(2.0f * t)));
+}
+
 __device__ __forceinline__ float activate(float z, int act) {
   if (act == 1) {
     const float r = fmaxf(z, 0.f);

@@ -173,8 +173,10 @@ class Engine:
 
     def _layout(self, entries, total, all_rows):
         """Host arrays of a step: the entries' order among the rows, and every entry's first row."""
-        order = sorted(range(len(entries)), key=lambda i: len(entries[i].tokens) > 1)   # stable: single rows first
         loc = self.cache.allocator.alloc(total)
+        if total == len(entries):
+            return self._layout_singles(entries, loc, all_rows)
+        order = sorted(range(len(entries)), key=lambda i: len(entries[i].tokens) > 1)   # stable: single rows first
         ids, pos, row_seq, row_req, first = [], [], [], [], {}
         row0, rows, start, slot, tile0, tile_row, tile_rows = [], [], [], [], [], [], []
         r = singles = 0
@@ -207,6 +209,22 @@ class Engine:
                     row0=i32(row0), rows=i32(rows), start=i32(start), slot=i32(slot), tile0=i32(tile0), tile_row=i32(tile_row),
                     tile_rows=i32(tile_rows), logit_rows=i32(want))
         return StepBatch(host, singles, self.req_to_token, self.max_context), first
+
+    def _layout_singles(self, entries, loc, all_rows):
+        """The same for a step of single rows (every decode step)."""
+        n = len(entries)
+        seqs = [e.seq for e in entries]
+        at = np.asarray([s.length for s in seqs], dtype=np.int32)
+        slot = np.asarray([s.slot for s in seqs], dtype=np.int32)
+        rows, none = np.arange(n, dtype=np.int32), np.zeros(0, dtype=np.int32)
+        for s, one in zip(seqs, loc.split(1)):
+            s.locs.append(one)
+            s.length += 1
+        want = rows if all_rows else np.asarray([i for i, e in enumerate(entries) for _ in e.want], dtype=np.int32)
+        host = dict(ids=np.asarray([e.tokens[0] for e in entries], dtype=np.int32), positions=at, loc=loc.numpy().astype(np.int32),
+                    row_seq=rows, row_req=slot, row0=rows, rows=np.ones(n, dtype=np.int32), start=at, slot=slot,
+                    tile0=np.zeros(n, dtype=np.int32), tile_row=none, tile_rows=none, logit_rows=want)
+        return StepBatch(host, n, self.req_to_token, self.max_context), dict(enumerate(range(n)))
 
     def _forward(self, batch, collect=None):
         assign_slots(self.req_to_token, batch.seqs.row_seq, batch.seqs.slot, batch.positions, batch.loc)

@@ -15,8 +15,9 @@ class FeedForward:
         self.up = Linear(padded(up, ff, pitch))
         self.down = Linear(padded(down, pitch, ff))
 
-    def linears(self):
-        return [self.up, self.down]
+    def bytes(self) -> int:
+        """Bytes of matrix weights one step reads."""
+        return sum(x.bytes() for x in (self.up, self.down))
 
     def forward(self, h):
         src = self.up.source(h)

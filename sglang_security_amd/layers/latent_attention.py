@@ -55,8 +55,9 @@ class LatentAttention:
                                        padded(uvh, H, self.vp, self.Rp).view(H * self.vp, self.Rp)]).contiguous()
         self.o = Linear(padded(o, pitch, self.op))
 
-    def linears(self):
-        return [self.down, self.uq, self.o]
+    def bytes(self) -> int:
+        """Bytes of matrix weights one step reads."""
+        return sum(x.bytes() for x in (self.down, self.uq, self.o)) + sum(t.numel() * t.element_size() for t in (self.wk, self.wv))
 
     @property
     def cache_row(self):
@@ -76,16 +77,16 @@ class LatentAttention:
         qa = torch.empty(M, H, self.Rp + self.rotp, dtype=self.dtype, device=q.device)
         hops.head_gemm(q[..., : self.kp], self.wk, qa[..., : self.Rp], self.kp, self.Rp)
         hops.latent_rope_q(q[..., self.kp:], qa[..., self.Rp:], self.cos_sin, pos, self.rot_dims)
+        mixed = torch.empty(M, H, self.Rp, dtype=self.dtype, device=q.device)
         if tiles:
             S = self._splits(M, batch.max_context)
             part = torch.empty(M, H, S, self.Rp, dtype=torch.float32, device=q.device)
             lse = torch.empty(M, H, S, dtype=torch.float32, device=q.device)
             hops.latent_decode(qa, pool, batch.req_to_token, req, pos, part, lse, self.Rp, self.window, self.scale)
-            hops.head_gemm(part, self.wv, attn, self.Rp, self.vn, lse=lse)
+            hops.latent_merge(part, lse, mixed)
         else:
-            mixed = torch.empty(M, H, self.Rp, dtype=self.dtype, device=q.device)
             hops.latent_attention_rows(qa, pool, batch.req_to_token, req, pos, mixed, self.window, self.scale)
-            hops.head_gemm(mixed, self.wv, attn, self.Rp, self.vn)
+        hops.head_gemm(mixed, self.wv, attn, self.Rp, self.vn)
 
     def _expanded(self, q, batch, pool, out):
         """Rows from batch.singles on: q, out are the whole step's rows."""

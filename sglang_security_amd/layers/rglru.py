@@ -43,8 +43,9 @@ class Rglru:
                                    conv_b=f("conv.b"), wr=gates[0], wi=gates[1], br=f("ra.b"), bi=f("ri.b"), sp=channels(sp),
                                    blocks=self.blocks, bwp=self.bwp)
 
-    def linears(self):
-        return [self.xy, self.o]
+    def bytes(self) -> int:
+        """Bytes of matrix weights one step reads."""
+        return sum(x.bytes() for x in (self.xy, self.o)) + sum(t.numel() * t.element_size() for t in (self.w.wr, self.w.wi))
 
     def forward(self, h, batch, cache):
         """cache: the layer's mem_cache.RecurrentStatePool.  Returns the output product's source."""

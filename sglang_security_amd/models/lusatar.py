@@ -47,39 +47,59 @@ def layer_runs(layers: int, loop: Optional[dict]) -> List[LayerRun]:
     return runs
 
 
-class _Layer:
-    """Weights of one layer."""
-
-    def __init__(self, model: "Lusatar", i: int, c: dict, weights):
-        D, pitch = model.width, model.pitch
+def tensor_shapes(config: dict) -> dict:
+    """Shape of every tensor of a checkpoint with this configuration, by name."""
+    D, loop = config["width"], config.get("loop")
+    out = {"embed": (config["vocab"], D), "final.norm": (D,)}
+    if loop:
+        out["loop.step"] = (loop["times"], D)
+    for i, c in enumerate(config["layers"]):
         m = c["mixer"]
-        norm = lambda n: vector(weights.get(f"l{i}.{n}", (D,), torch.float32), pitch)
-        self.kind = c["type"]
-        self.norm1, self.norm1b = norm("norm1"), norm("norm1b")
-        if self.kind == "latent_attention":
-            H, R, hd = m["heads"], m["kv_rank"], m["dim"] + m["rot_dim"]
-            shapes = {"dq": (m["q_rank"], D), "dq.norm": (m["q_rank"],), "uq": (H * hd, m["q_rank"]),
-                      "dkv": (R + m["rot_dim"], D), "dkv.norm": (R,), "uk": (H * m["dim"], R), "uv": (H * m["vdim"], R),
-                      "o": (D, H * m["vdim"])}
-            rot = m["rot"]
-            table = model.rotary(rot["dims"], rot["base"], rot.get("scaling"))
-            self.mixer = LatentAttention(m, lambda n: weights.get(f"l{i}.mix.{n}", shapes[n]), pitch, model.eps, model.dtype,
-                                         model.device, table)
-        elif self.kind == "rglru":
+        if c["type"] == "latent_attention":
+            H, R = m["heads"], m["kv_rank"]
+            mix = {"dq": (m["q_rank"], D), "dq.norm": (m["q_rank"],), "uq": (H * (m["dim"] + m["rot_dim"]), m["q_rank"]),
+                   "dkv": (R + m["rot_dim"], D), "dkv.norm": (R,), "uk": (H * m["dim"], R), "uv": (H * m["vdim"], R),
+                   "o": (D, H * m["vdim"])}
+        elif c["type"] == "rglru":
             W, nb = m["width"], m["blocks"]
+            if W % nb:
+                raise ValueError(f"layer {i}: {W} channels in {nb} blocks")
             bw = W // nb
-            shapes = {"y": (W, D), "y.b": (W,), "x": (W, D), "x.b": (W,), "conv": (W, m["conv"]), "conv.b": (W,),
-                      "ra": (nb, bw, bw), "ra.b": (nb, bw), "ri": (nb, bw, bw), "ri.b": (nb, bw), "lam": (W,), "o": (D, W)}
-            self.mixer = Rglru(m, lambda n: weights.get(f"l{i}.mix.{n}", shapes[n]), pitch, model.dtype)
+            mix = {"y": (W, D), "y.b": (W,), "x": (W, D), "x.b": (W,), "conv": (W, m["conv"]), "conv.b": (W,), "ra": (nb, bw, bw),
+                   "ra.b": (nb, bw), "ri": (nb, bw, bw), "ri.b": (nb, bw), "lam": (W,), "o": (D, W)}
         else:
-            raise ValueError(f"layer {i}: unknown mixer {self.kind!r}")
-        self.mlp = None
+            raise ValueError(f"layer {i}: unknown mixer {c['type']!r}")
+        out.update({f"l{i}.mix.{k}": s for k, s in mix.items()})
+        norms = ["norm1", "norm1b"]
         if c.get("mlp"):
             if c["mlp"]["kind"] != "dense":
                 raise ValueError(f"layer {i}: unknown feed-forward {c['mlp']['kind']!r}")
             ff = c["mlp"]["ff"]
+            out[f"l{i}.mlp.up"], out[f"l{i}.mlp.down"] = (ff, D), (D, ff)
+            norms += ["norm2", "norm2b"]
+        out.update({f"l{i}.{n}": (D,) for n in norms})
+    return out
+
+
+class _Layer:
+    """Weights of one layer."""
+
+    def __init__(self, model: "Lusatar", i: int, c: dict, get):
+        pitch, m = model.pitch, c["mixer"]
+        norm = lambda n: vector(get(f"l{i}.{n}", torch.float32), pitch)
+        mix = lambda n: get(f"l{i}.mix.{n}")
+        self.kind = c["type"]
+        self.norm1, self.norm1b = norm("norm1"), norm("norm1b")
+        if self.kind == "latent_attention":
+            rot = m["rot"]
+            self.mixer = LatentAttention(m, mix, pitch, model.eps, model.dtype, model.device,
+                                         model.rotary(rot["dims"], rot["base"], rot.get("scaling")))
+        else:
+            self.mixer = Rglru(m, mix, pitch, model.dtype)
+        self.mlp = None
+        if c.get("mlp"):
             self.norm2, self.norm2b = norm("norm2"), norm("norm2b")
-            self.mlp = FeedForward(weights.get(f"l{i}.mlp.up", (ff, D)), weights.get(f"l{i}.mlp.down", (D, ff)), pitch)
+            self.mlp = FeedForward(get(f"l{i}.mlp.up"), get(f"l{i}.mlp.down"), pitch)
 
     def cache_spec(self):
         if self.kind == "latent_attention":
@@ -88,6 +108,8 @@ class _Layer:
 
 
 class Lusatar:
+    tensor_shapes = staticmethod(tensor_shapes)
+
     def __init__(self, config: dict, weights, dtype: torch.dtype, device, max_context: int):
         if dtype not in (torch.bfloat16, torch.float32):
             raise ValueError("Lusatar runs in bfloat16 or float32")
@@ -97,17 +119,19 @@ class Lusatar:
         self.embed_scale = config["embedding"]["scale"]
         self.logit_cap = config.get("logit_softcap")
         self._tables = {}
-        table = padded(weights.get("embed", (self.vocab, self.width)), pad(self.vocab, 16), self.pitch)
+        shapes = tensor_shapes(config)
+        get = lambda name, dt=None: weights.get(name, shapes[name], dt)
+        table = padded(get("embed"), pad(self.vocab, 16), self.pitch)
         self.head = Linear(table)                         # the row-major copy is also the embedding table
-        self.layers = [_Layer(self, i, c, weights) for i, c in enumerate(config["layers"])]
+        self.layers = [_Layer(self, i, c, get) for i, c in enumerate(config["layers"])]
         loop = config.get("loop")
         self.runs = layer_runs(len(self.layers), loop)
         self.loop_step = None
-        if loop and any(r.opens is not None for r in self.runs):
-            steps = weights.get("loop.step", (loop["times"], self.width), torch.float32)
+        if loop:
+            steps = get("loop.step", torch.float32)
             self.loop_step = [vector(s, self.pitch) for s in steps]
         self.repeats = any(r.opens for r in self.runs)    # a pass after the first: the embedding output is kept
-        self.final_norm = vector(weights.get("final.norm", (self.width,), torch.float32), self.pitch)
+        self.final_norm = vector(get("final.norm", torch.float32), self.pitch)
         self._tables.clear()
 
     def rotary(self, dims, base, scaling):
@@ -122,7 +146,7 @@ class Lusatar:
 
     def weight_bytes(self) -> int:
         """Bytes of matrix weights a step over all layer runs reads."""
-        per = [sum(x.bytes() for x in L.mixer.linears() + (L.mlp.linears() if L.mlp else [])) for L in self.layers]
+        per = [L.mixer.bytes() + (L.mlp.bytes() if L.mlp else 0) for L in self.layers]
         return sum(per[r.layer] for r in self.runs) + self.head.bytes()
 
     def forward(self, batch, cache, collect: Optional[list] = None):

@@ -150,20 +150,27 @@ def latent_rope_q(src, out, cos_sin, positions, rot_dims):
                                    _stream(src)), "latent_rope_q")
 
 
-def head_gemm(a, w, out, K, Np, lse=None):
-    """out [M, H, N] = a [M, H, K] . w^T per head; with `lse` [M, H, S], a holds split partials [M, H, S, K]."""
+def head_gemm(a, w, out, K, Np):
+    """out [M, H, N] = a [M, H, K] . w^T per head."""
     M, H, N = out.shape
     _need_gpu(a, w, out)
-    if a.shape[0] != M or a.shape[1] != H or a.shape[-1] < K or a.stride(-1) != 1 or out.stride(2) != 1 or w.numel() != H * Np * K:
+    if a.shape[0] != M or a.shape[1] != H or a.shape[2] < K or a.stride(2) != 1 or out.stride(2) != 1 or w.numel() != H * Np * K:
         raise SglkError("head_gemm: shapes do not match")
-    if lse is not None and (a.dtype != torch.float32 or not a.is_contiguous() or a.shape[3] != K or
-                            lse.shape != a.shape[:3] or lse.dtype != torch.float32 or not lse.is_contiguous()):
-        raise SglkError("head_gemm: split partials must be contiguous float32")
-    if lse is None and a.dtype != out.dtype:
-        raise SglkError("head_gemm: a and out must be of one type")
-    check(lib().sglk_head_gemm(_ptr(a), _ptr(lse), 1 if lse is None else lse.shape[2], a.stride(0), a.stride(1), _ptr(w),
-                               _ptr(out), M, H, N, Np, K, out.stride(0), out.stride(1), dtype_code(out.dtype), _stream(out)),
-          "head_gemm")
+    if not (a.dtype == out.dtype == w.dtype):
+        raise SglkError("head_gemm: a, w and out must be of one type")
+    check(lib().sglk_head_gemm(_ptr(a), a.stride(0), a.stride(1), _ptr(w), _ptr(out), M, H, N, Np, K, out.stride(0), out.stride(1),
+                               dtype_code(out.dtype), _stream(out)), "head_gemm")
+    return out
+
+
+def latent_merge(part, lse, out):
+    """Split partials [M, H, S, K] and their log-sum-exps [M, H, S] -> out [M, H, K] contiguous."""
+    M, H, S, K = part.shape
+    _f32(part, M * H * S * K, "latent_merge: part")
+    _f32(lse, M * H * S, "latent_merge: lse")
+    if out.shape != (M, H, K) or not out.is_contiguous():
+        raise SglkError("latent_merge: out must be contiguous [M, H, K]")
+    check(lib().sglk_latent_merge(_ptr(part), _ptr(lse), S, _ptr(out), M * H, K, dtype_code(out.dtype), _stream(out)), "latent_merge")
     return out
 
 

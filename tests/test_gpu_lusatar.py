@@ -129,7 +129,7 @@ def test_latent_prep_and_query_rotation(dtype, splits, q_rank, R, rot_dim, rot_d
 
 
 @pytest.mark.parametrize("M_,H_,N,K", [(1, 3, 20, 64), (64, 2, 512, 128), (70, 5, 128, 512), (130, 1, 36, 448)])
-def test_head_gemm(M_, H_, N, K):
+def test_head_products_and_merge(M_, H_, N, K):
     from sglang_security_amd import ops_hybrid as H
     from sglang_security_amd.layers.linear import pad, padded
 
@@ -149,9 +149,9 @@ def test_head_gemm(M_, H_, N, K):
     part[:, :, 2] = math.nan
     wt = torch.softmax(lse.double(), -1)
     merged = (wt[..., None] * torch.nan_to_num(part.double())).sum(2)
-    out.zero_()
-    H.head_gemm(part.to(DEV), wp, out, K, Np, lse=lse.to(DEV))
-    close(out, torch.einsum("mhk,hnk->mhn", merged, w.double()), 1e-2, "merged")
+    for dt in (BF16, F32):
+        got = torch.empty(M_, H_, K, dtype=dt, device=DEV)
+        close(H.latent_merge(part.to(DEV), lse.to(DEV), got), merged, TOL[dt], "merged")
 
 
 def _pool_case(g, lengths, Rp, rotp, R, rot, dtype, loud=()):
@@ -196,13 +196,12 @@ def test_latent_decode(H_, R, rot, window):
         want[b] = o[-1]
     req, pos = i32(*range(1, len(lengths) + 1)), i32(*[n - 1 for n in lengths])
     args = (q.to(DEV), pool.to(DEV), r2t.to(DEV), req, pos)
-    ident = H.pack_heads(torch.eye(Rp).expand(H_, Rp, Rp).contiguous().to(BF16)).to(DEV)
     for S in (1, 3, 8):
         part = torch.full((len(lengths), H_, S, Rp), math.nan, device=DEV)
         lse = torch.full((len(lengths), H_, S), math.nan, device=DEV)
         H.latent_decode(*args, part, lse, Rp, window, scale)
         out = torch.empty(len(lengths), H_, Rp, dtype=BF16, device=DEV)
-        H.head_gemm(part, ident, out, Rp, Rp, lse=lse)
+        H.latent_merge(part, lse, out)
         close(out, want, 1e-2, f"{S} splits")
     for dt, tol in ((BF16, 1e-2), (F32, 1e-5)):
         out = torch.empty(len(lengths), H_, Rp, dtype=dt, device=DEV)
