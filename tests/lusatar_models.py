@@ -40,6 +40,9 @@ CONFIGS = {
     # one pass of a loop at the end, wide heads
     "tail": config([recurrent(width=72, blocks=6), attention(heads=2, dim=72, rot_dim=40, vdim=136, kv_rank=150, size=40)],
                    width=64, vocab=100, loop={"start": 1, "stop": 2, "times": 1}, cap=30.0, eps=1e-3),
+    # sizes no tile kernel takes, odd widths, a loop that runs nothing extra
+    "large": config([attention(heads=2, dim=260, rot_dim=72, vdim=300, kv_rank=530, size=33, ff=33), recurrent(width=1056, blocks=1)],
+                    width=50, vocab=77, loop={"start": 1, "stop": 1, "times": 2}),
 }
 
 
