@@ -6,13 +6,13 @@ import math
 
 import torch
 
-YARN = {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}
+YARN = {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}
 
 
 def _lusatar(width, heads, q_rank, ff, blocks, groups, vocab, window, loop=None):
     att = {"type": "latent_attention",
            "mixer": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": q_rank, "kv_rank": 512, "mask": {"size": window},
-                     "rot": {"base": 50000.0, "dims": 64, "scaling": YARN}, "scale": 1 / math.sqrt(192)},
+                     "rot": {"base": 100000.0, "dims": 64, "scaling": YARN}, "scale": 1 / math.sqrt(192)},
            "mlp": {"kind": "dense", "ff": ff}}
     rec = {"type": "rglru", "mixer": {"width": width, "blocks": blocks, "conv": 4}, "mlp": {"kind": "dense", "ff": ff}}
     return {"architecture": "Lusatar", "embedding": {"scale": math.sqrt(width)}, "layers": [rec, rec, att] * groups,

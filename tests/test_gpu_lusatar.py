@@ -96,7 +96,7 @@ def test_activations_and_capped_logits(dtype, splits):
 
 # ---- latent attention -----------------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("dtype,splits", [(BF16, 0), (BF16, 4), (F32, 1)])
-@pytest.mark.parametrize("q_rank,R,rot_dim,rot_dims", [(80, 96, 16, 16), (28, 36, 8, 4), (1536, 512, 64, 64), (130, 70, 70, 40)])
+@pytest.mark.parametrize("q_rank,R,rot_dim,rot_dims", [(72, 104, 24, 24), (28, 36, 8, 4), (1536, 512, 64, 64), (130, 70, 70, 40)])
 def test_latent_prep_and_query_rotation(dtype, splits, q_rank, R, rot_dim, rot_dims):
     from sglang_security_amd import ops_hybrid as H
     from sglang_security_amd.layers.linear import pad, vector
@@ -171,8 +171,8 @@ def _pool_case(g, lengths, Rp, rotp, R, rot, dtype, loud=()):
     return r2t, pool.to(dtype)
 
 
-@pytest.mark.parametrize("H_,R,rot", [(8, 96, 16), (16, 512, 64), (40, 512, 64), (3, 36, 8), (33, 200, 64), (1, 320, 64)])
-@pytest.mark.parametrize("window", [1, 21, 64, 96, None])
+@pytest.mark.parametrize("H_,R,rot", [(6, 104, 24), (16, 512, 64), (40, 512, 64), (3, 36, 8), (33, 200, 64), (1, 320, 64)])
+@pytest.mark.parametrize("window", [1, 21, 64, 90, None])
 def test_latent_decode(H_, R, rot, window):
     """Rows at, just inside and just outside the window's edge; one key stands out just inside or just outside."""
     from sglang_security_amd import ops_hybrid as H
@@ -209,9 +209,9 @@ def test_latent_decode(H_, R, rot, window):
         close(out, want, tol, f"rows {dt}")
 
 
-@pytest.mark.parametrize("H_,kp,vp,vdim", [(8, 64, 64, 64), (3, 128, 128, 128), (2, 64, 128, 70), (5, 192, 64, 20), (2, 256, 256, 250),
+@pytest.mark.parametrize("H_,kp,vp,vdim", [(6, 64, 64, 64), (3, 128, 128, 128), (2, 64, 128, 70), (5, 192, 64, 20), (2, 256, 256, 250),
                                            (1, 128, 256, 201), (2, 192, 256, 256), (2, 256, 64, 64), (2, 64, 256, 129)])
-@pytest.mark.parametrize("window", [1, 21, 64, 96, None])
+@pytest.mark.parametrize("window", [1, 21, 64, 90, None])
 def test_latent_prefill(H_, kp, vp, vdim, window):
     """Portions of unequal length behind prefixes of unequal length; loud keys inside and outside the windows."""
     from sglang_security_amd import ops_hybrid as H
@@ -286,7 +286,7 @@ class _Batch:
 
 
 @pytest.mark.parametrize("dtype", [F32, BF16])
-@pytest.mark.parametrize("width,blocks,taps", [(60, 3, 4), (64, 1, 1), (128, 2, 2), (128, 4, 4), (96, 8, 7), (512, 2, 4)])
+@pytest.mark.parametrize("width,blocks,taps", [(60, 3, 4), (64, 1, 1), (192, 2, 2), (128, 4, 4), (96, 8, 7), (512, 2, 4)])
 def test_rglru_portions_and_slots(dtype, width, blocks, taps):
     """Four sequences of which pieces of every length run together, slots reused for later sequences."""
     layer, cache, w, c = _rglru(width, blocks, taps, dtype)
