@@ -1011,10 +1011,13 @@ SGLK_API int sglk_residual_norm(float* x, const void* embed, const int32_t* ids,
                                 const float* w_post, float* x0, int add_x0, const float* step, const float* w_next, void* h,
                                 int64_t h_stride, const int32_t* rows, int store_x, int M, int width, int pitch, float eps,
                                 int dtype, void* stream);
-/* out[m][n] = act(src[m][n] + bias[n]); act: 0 none, 1 square of relu, 2 gelu (tanh form) */
+/* out[m][n] = act(src[m][n] + bias[n]); act: 0 none, 1 square of relu, 2 gelu (tanh form), 3 silu */
 SGLK_API int sglk_source_act(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
                              const float* bias, void* out, int M, int N, int64_t out_stride, int act, int dtype,
                              void* stream);
+/* out[m][n] = act(src[m][n]) * src[m][N + n] */
+SGLK_API int sglk_source_gated_act(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
+                                   void* out, int M, int N, int64_t out_stride, int act, int dtype, void* stream);
 /* fp32 logits [M, V] = cap * tanh(src / cap) (cap <= 0: src) */
 SGLK_API int sglk_capped_logits(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
                                 float* out, int M, int N, int V, int64_t out_stride, float cap, int dtype, void* stream);
@@ -1094,6 +1097,54 @@ SGLK_API int sglk_rglru_rows(const void* src, int src_f32, int splits, int64_t p
                              const void* wr, const void* wi, const float* br, const float* bi, const float* sp, float* da,
                              float* db, float* state, void* out, int64_t out_stride, int bwp, int blocks, int dtype,
                              void* stream);
+
+/* Causal grouped-query attention whose values are its keys before their norm (tied_attention.hip): a pool row holds a
+ * token's keys, kv_heads * D elements, rms[slot] the reciprocal root mean square of the whole row.  Scores are base 2:
+ * (q . row) * rms + bias[head][min(distance, nb - 1)]; sink[head] is one more term of the softmax's denominator.
+ * tied_prep: src columns [q_cols | k_cols] + bias -> q = x / rms(x over q_size) * wq * factor[position]; key rows (with
+ * their bias) and their reciprocal root mean squares into pool and rms at loc. */
+SGLK_API int sglk_tied_prep(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
+                            const float* bias, const float* wq, const float* factor, void* q, void* pool,
+                            int64_t pool_stride, float* rms, const int32_t* loc, const int32_t* positions, int M, int q_cols,
+                            int k_cols, int q_size, int k_size, float eps, int dtype, void* stream);
+SGLK_API int sglk_tied_supported(int D);
+/* bf16 rows of one token each over positions [0, p] of request req[m]: normalised partials part [M][H][splits][D], lse
+ * base 2 (-inf: empty split), without the sink */
+SGLK_API int sglk_tied_decode(const void* q, const void* pool, int64_t pool_stride, const float* rms,
+                              const int32_t* req_to_token, int64_t r2t_stride, const float* bias, int nb, const float* sink,
+                              int H, int kv_heads, int D, const int32_t* req, const int32_t* positions, float* part,
+                              float* lse, int M, int splits, void* stream);
+/* out[m][h * D ..] = out_scale * the merged partials, the sink counted */
+SGLK_API int sglk_tied_merge(const float* part, const float* lse, const float* sink, int splits, float out_scale, void* out,
+                             int64_t out_stride, int M, int H, int D, int dtype, void* stream);
+/* bf16 runs of rows: sequence b has rows[b] rows from row0[b] on, the first one at position start[b], of request req[b] */
+SGLK_API int sglk_tied_prefill(const void* q, const void* pool, int64_t pool_stride, const float* rms,
+                               const int32_t* req_to_token, int64_t r2t_stride, const float* bias, int nb, const float* sink,
+                               int H, int kv_heads, int D, const int32_t* row0, const int32_t* rows, const int32_t* start,
+                               const int32_t* req, int n_seqs, int max_rows, float out_scale, void* out,
+                               int64_t out_stride, void* stream);
+/* finished rows, any size and float type (one wave per row and head) */
+SGLK_API int sglk_tied_rows(const void* q, const void* pool, int64_t pool_stride, const float* rms,
+                            const int32_t* req_to_token, int64_t r2t_stride, const float* bias, int nb, const float* sink,
+                            int H, int kv_heads, int D, const int32_t* req, const int32_t* positions, float out_scale,
+                            void* out, int64_t out_stride, int M, int dtype, void* stream);
+
+/* u = act(causal convolution of src + bias), act 0 or 3; conv [taps][W], conv_state [slots][taps - 1][W] of the activation
+ * type (short_conv.h); sequences as for rglru_conv, sequence m < singles is row m */
+SGLK_API int sglk_short_conv(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride,
+                             const float* bias, const float* conv, const float* conv_b, void* u, void* conv_state,
+                             const int32_t* row_seq, const int32_t* row0, const int32_t* rows, const int32_t* start,
+                             const int32_t* slot, int M, int W, int taps, int singles, int n_seqs, int act, int dtype,
+                             void* stream);
+/* The gated delta rule (delta_rule.hip): u columns [kv_heads * dp queries | kv_heads * dp keys | heads * vp values]; src
+ * columns [heads * vp gates | b_col: heads step sizes | a_col: heads decays], before their activations; state
+ * [slots][heads][dp][vp]; out rows of heads * vp.  Sequences seq0 .. n_seqs - 1. */
+SGLK_API int sglk_delta_step(const void* u, int64_t u_stride, const void* src, int src_f32, int splits, int64_t part_stride,
+                             int64_t src_stride, int b_col, int a_col, const float* rate, const float* dt,
+                             const float* norm, float* state, void* out, int64_t out_stride, const int32_t* row_seq,
+                             const int32_t* row0, const int32_t* rows, const int32_t* start, const int32_t* slot, int M,
+                             int kv_heads, int heads, int dp, int vp, int dim, int vdim, float out_scale, float eps,
+                             int seq0, int n_seqs, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

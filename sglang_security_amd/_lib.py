@@ -132,6 +132,7 @@ _SIGS = {
     "sglk_residual_norm": (i32, [p, p, p, i64, f32, p, i32, i32, i64, i64, p, p, i32, p, p, p, i64, p, i32, i32,
         i32, i32, f32, i32, p]),
     "sglk_source_act": (i32, [p, i32, i32, i64, i64, p, p, i32, i32, i64, i32, i32, p]),
+    "sglk_source_gated_act": (i32, [p, i32, i32, i64, i64, p, i32, i32, i64, i32, i32, p]),
     "sglk_capped_logits": (i32, [p, i32, i32, i64, i64, p, i32, i32, i32, i64, f32, i32, p]),
     "sglk_assign_slots": (i32, [p, i64, p, p, p, p, i32, p]),
     "sglk_latent_prep": (i32, [p, i32, i32, i64, i64, p, p, p, i64, p, i64, p, p, p, i32, i32, i32, i32, i32,
@@ -156,6 +157,15 @@ _SIGS = {
     "sglk_rglru_apply": (i32, [p, p, p, p, p, i64, p, p, p, i32, i32, i32, i32, i32, p]),
     "sglk_rglru_rows": (i32, [p, i32, i32, i64, i64, p, p, p, p, p, p, p, p, p, p, p, p, i32, i32, i32, i32,
         i32, p, p, p, p, p, p, p, p, p, i64, i32, i32, i32, p]),
+    "sglk_tied_prep": (i32, [p, i32, i32, i64, i64] + [p] * 5 + [i64] + [p] * 3 + [i32] * 5 + [f32, i32, p]),
+    "sglk_tied_supported": (i32, [i32]),
+    "sglk_tied_decode": (i32, [p, p, i64, p, p, i64, p, i32, p, i32, i32, i32, p, p, p, p, i32, i32, p]),
+    "sglk_tied_merge": (i32, [p, p, p, i32, f32, p, i64, i32, i32, i32, i32, p]),
+    "sglk_tied_prefill": (i32, [p, p, i64, p, p, i64, p, i32, p, i32, i32, i32, p, p, p, p, i32, i32, f32, p, i64, p]),
+    "sglk_tied_rows": (i32, [p, p, i64, p, p, i64, p, i32, p, i32, i32, i32, p, p, f32, p, i64, i32, i32, p]),
+    "sglk_short_conv": (i32, [p, i32, i32, i64, i64] + [p] * 10 + [i32] * 7 + [p]),
+    "sglk_delta_step": (i32, [p, i64, p, i32, i32, i64, i64, i32, i32, p, p, p, p, p, i64] + [p] * 5 + [i32] * 7 +
+                        [f32, f32, i32, i32, i32, p]),
     "sglk_ar_meta_size": (i64, []),
     "sglk_ar_init": (i64, [p, i32, i32, i32, i64]),
     "sglk_ar_init_handles": (i64, [p, p, i64, p, p, i32, i32, i32, i64]),

@@ -12,6 +12,7 @@ import os
 import shutil
 import subprocess
 import sys
+import zlib
 
 PKG = os.path.dirname(os.path.abspath(__file__))
 ROOT = os.path.dirname(PKG)
@@ -70,13 +71,9 @@ def build(force: bool = False, jobs: int = 6) -> str:
     return LIB
 
 
-# what the checkpoint-loaded models of the engine launch, and nothing else
-ENGINE = ("core.hip", "elementwise.hip", "gemm_dense.hip", "sampling.hip", "latent_attention.hip", "residual_norm.hip", "rglru.hip")
-
-
 def ensure(names, jobs: int = 8) -> str:
-    """Without a full library beside the package: compile the named sources into a library of their own (once; other
-    processes wait for the one that compiles) and make this process load that."""
+    """Without a full library beside the package: compile the named sources (models.kernel_sources) into a library of
+    their own (once; other processes wait for the one that compiles) and make this process load that."""
     from . import _lib
 
     if os.environ.get("SGLK_LIB") or os.path.exists(LIB):
@@ -84,7 +81,7 @@ def ensure(names, jobs: int = 8) -> str:
     import fcntl
 
     os.makedirs(OBJ, exist_ok=True)
-    part = os.path.join(PKG, "libsglk_engine.so")
+    part = os.path.join(PKG, f"libsglk_{zlib.crc32(' '.join(sorted(names)).encode()):08x}.so")
     with open(os.path.join(OBJ, ".lock"), "w") as lock:
         fcntl.flock(lock, fcntl.LOCK_EX)
         with cf.ThreadPoolExecutor(max_workers=jobs) as ex:

@@ -18,8 +18,10 @@ import sys
 def _generate(args) -> int:
     import torch
 
+    from . import build
     from .engine import Engine, SamplingParams, Scheduler
-    from .models import load_model
+    from .model_loader import load_config
+    from .models import SAMPLING_SOURCES, kernel_sources, load_model
 
     if not torch.cuda.is_available():
         raise SystemExit("no GPU (there is no CPU fallback)")
@@ -30,6 +32,7 @@ def _generate(args) -> int:
     if not prompts:
         raise SystemExit("no prompts")
     params = SamplingParams(args.max_new_tokens, args.temperature, args.top_k, args.top_p, args.min_p, tuple(args.stop or ()))
+    build.ensure(kernel_sources(load_config(args.model)) + SAMPLING_SOURCES)
     dev = torch.device("cuda", args.device)
     torch.cuda.set_device(dev)
     longest = max(len(p) for p in prompts) + args.max_new_tokens

@@ -143,6 +143,23 @@ __global__ void __launch_bounds__(256) source_act_kernel(RowSource src, const fl
   st8<T>(out, (int64_t)m * out_stride + n, v);
 }
 
+// out[m][n] = act(src[m][n]) * src[m][N + n]: gate columns, then as many others
+template <typename T>
+__global__ void __launch_bounds__(256) source_gated_act_kernel(RowSource src, void* __restrict__ out, int M, int N,
+                                                               int64_t out_stride, int act) {
+  const int nv = N / 8;
+  const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (idx >= (int64_t)M * nv) return;
+  const int m = (int)(idx / nv), n = (int)(idx - (int64_t)m * nv) * 8;
+  float v[8], w[8];
+  source8<T>(src, m, n, v);
+  source8<T>(src, m, N + n, w);
+#pragma unroll
+  for (int j = 0; j < 8; ++j)
+    v[j] = w[j] * (sizeof(typename Raw<T>::type) == 2 && act == 3 ? silu_fast(v[j]) : activate(v[j], act));
+  st8<T>(out, (int64_t)m * out_stride + n, v);
+}
+
 // logits[m][n] = cap * tanh(src[m][n] / cap) in fp32 (cap <= 0: as they are)
 template <typename T>
 __global__ void __launch_bounds__(256) capped_logits_kernel(RowSource src, float* __restrict__ out, int M, int N, int V,
@@ -220,7 +237,7 @@ int sglk_residual_norm(float* x, const void* embed, const int32_t* ids, int64_t 
 int sglk_source_act(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride, const float* bias,
                     void* out, int M, int N, int64_t out_stride, int act, int dtype, void* stream) {
   SGLK_CHECK(M >= 0 && N > 0 && N % 8 == 0 && out_stride % 8 == 0 && out_stride >= N, "source_act: bad shape");
-  SGLK_CHECK(act >= 0 && act <= 2, "source_act: act is 0 (none), 1 (square of relu) or 2 (gelu, tanh form)");
+  SGLK_CHECK(act >= 0 && act <= 3, "source_act: act is 0 (none), 1 (square of relu), 2 (gelu, tanh form) or 3 (silu)");
   if (M == 0) return SGLK_OK;
   SGLK_CHECK(src && out && aligned16(out), "source_act: null or unaligned pointer");
   if (int rc = check_source(src, src_f32, splits, part_stride, src_stride, N, dtype, "source_act")) return rc;
@@ -229,6 +246,22 @@ int sglk_source_act(const void* src, int src_f32, int splits, int64_t part_strid
                       hipLaunchKernelGGL((source_act_kernel<T>), dim3((unsigned)((vecs + 255) / 256)), dim3(256), 0,
                                          (hipStream_t)stream, RowSource{src, src_f32, splits, part_stride, src_stride}, bias,
                                          out, M, N, out_stride, act));
+  SGLK_LAUNCH_CHECK();
+  return SGLK_OK;
+}
+
+int sglk_source_gated_act(const void* src, int src_f32, int splits, int64_t part_stride, int64_t src_stride, void* out, int M,
+                          int N, int64_t out_stride, int act, int dtype, void* stream) {
+  SGLK_CHECK(M >= 0 && N > 0 && N % 8 == 0 && out_stride % 8 == 0 && out_stride >= N, "source_gated_act: bad shape");
+  SGLK_CHECK(act >= 0 && act <= 3, "source_gated_act: act is 0 (none), 1 (square of relu), 2 (gelu, tanh form) or 3 (silu)");
+  if (M == 0) return SGLK_OK;
+  SGLK_CHECK(src && out && aligned16(out), "source_gated_act: null or unaligned pointer");
+  if (int rc = check_source(src, src_f32, splits, part_stride, src_stride, 2 * N, dtype, "source_gated_act")) return rc;
+  const int64_t vecs = (int64_t)M * (N / 8);
+  SGLK_DISPATCH_FLOAT(dtype, T,
+                      hipLaunchKernelGGL((source_gated_act_kernel<T>), dim3((unsigned)((vecs + 255) / 256)), dim3(256), 0,
+                                         (hipStream_t)stream, RowSource{src, src_f32, splits, part_stride, src_stride}, out, M,
+                                         N, out_stride, act));
   SGLK_LAUNCH_CHECK();
   return SGLK_OK;
 }

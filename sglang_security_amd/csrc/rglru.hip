@@ -25,6 +25,7 @@
 #include "attention_tile.h"
 #include "common.h"
 #include "row_source.h"
+#include "short_conv.h"
 
 namespace sglk {
 
@@ -32,16 +33,6 @@ constexpr int kScanTile = 64;
 constexpr int kGateMaxBlock = 1024;
 constexpr int gate_lds(int bwp) { return kScanTile * (bwp * 2 + 16); }
 
-struct RecurrentSeqs {
-  const int32_t* row_seq;  // sequence of a row
-  const int32_t* row0;     // first row of a sequence
-  const int32_t* rows;     // number of its rows
-  const int32_t* start;    // position of its first row
-  const int32_t* slot;     // its state slot
-};
-
-__device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
 // decay and input weight of a channel from its two gate pre-activations and softplus(lambda)
 __device__ __forceinline__ void gate_terms(float zr, float zi, float sp, float u, float& a, float& b) {
@@ -63,26 +54,11 @@ __device__ __forceinline__ void gate_terms_fast(float zr, float zi, float nbr, f
   b = __builtin_amdgcn_sqrtf(x > -0.03f ? near : fmaf(-a, a, 1.0f)) * si * u;
 }
 
-struct RglruConv {
-  RowSource src;          // columns [0, W) x branch, [W, 2 W) y branch
-  const float* bx;        // [W]
-  const float* by;
-  const float* conv;      // [taps][W], last tap: the row itself
-  const float* conv_b;
-  void* u;                // [rows, W]
-  void* y;
-  void* state;            // [slots][taps - 1][W], of the activation type
-  RecurrentSeqs seq;
-  int M, W, taps, singles;
+// the convolution of the x branch (columns [0, W) of its source) beside the y branch (columns [W, 2 W))
+struct RglruConv : ShortConv {
+  const float* by;        // [W]
+  void* y;                // [rows, W]
 };
-
-// convolution input of row m: the x branch with its bias, as the activation type holds it
-template <typename T>
-__device__ __forceinline__ void conv_input8(const RglruConv& a, int m, int c, const float (&bias)[8], float (&x)[8]) {
-  source8<T>(a.src, m, c, x);
-#pragma unroll
-  for (int j = 0; j < 8; ++j) x[j] = round_to<T>(x[j] + bias[j]);
-}
 
 // One thread: eight channels of R rows; blockIdx.y 0: the x branch, 1: the y branch.
 template <typename T, int R>
@@ -91,97 +67,21 @@ __global__ void __launch_bounds__(256) rglru_conv_kernel(RglruConv a) {
   const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (idx >= (int64_t)((a.M + R - 1) / R) * nv) return;
   const int m0 = (int)(idx / nv) * R, c = (int)(idx % nv) * 8;
-  float bias[8], acc[8];
-  if (blockIdx.y) {
-    ld8<float>(a.by, c, bias);
-#pragma unroll
-    for (int r = 0; r < R; ++r) {
-      const int m = m0 + r;
-      if (m >= a.M) break;
-      source8<T>(a.src, m, a.W + c, acc);
-#pragma unroll
-      for (int j = 0; j < 8; ++j)
-        acc[j] = sizeof(typename Raw<T>::type) == 4 ? gelu_tanh(acc[j] + bias[j]) : gelu_tanh_fast(acc[j] + bias[j]);
-      st8<T>(a.y, (int64_t)m * a.W + c, acc);
-    }
+  if (blockIdx.y == 0) {
+    short_conv_rows<T, R, 0>(a, m0, c);
     return;
   }
-  ld8<float>(a.bx, c, bias);
-  const int keep = a.taps - 1;
-  if constexpr (R > 1) {
-    // four taps, rows of one sequence with everything they need in this step: every input is formed once
-    const int s = a.seq.row_seq[m0];
-    if (keep == 3 && m0 + R <= a.M && a.seq.row_seq[m0 + R - 1] == s && m0 - a.seq.row0[s] >= 3) {
-      float x[R + 3][8], w[4][8], cb[8];
+  float bias[8], acc[8];
+  ld8<float>(a.by, c, bias);
 #pragma unroll
-      for (int r = 0; r < R + 3; ++r) conv_input8<T>(a, m0 - 3 + r, c, bias, x[r]);
+  for (int r = 0; r < R; ++r) {
+    const int m = m0 + r;
+    if (m >= a.M) break;
+    source8<T>(a.src, m, a.W + c, acc);
 #pragma unroll
-      for (int t = 0; t < 4; ++t) ld8<float>(a.conv, (int64_t)t * a.W + c, w[t]);
-      ld8<float>(a.conv_b, c, cb);
-#pragma unroll
-      for (int r = 0; r < R; ++r) {
-#pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          acc[j] = cb[j];
-#pragma unroll
-          for (int t = 0; t < 4; ++t) acc[j] = fmaf(x[r + t][j], w[t][j], acc[j]);
-        }
-        st8<T>(a.u, (int64_t)(m0 + r) * a.W + c, acc);
-      }
-      return;
-    }
-  }
-  for (int m = m0; m < min(m0 + R, a.M); ++m) {
-    const int s = a.seq.row_seq[m];
-    const int start = a.seq.start[s];
-    const int k = m - a.seq.row0[s];  // row within its sequence's portion
-    const int64_t st0 = (int64_t)a.seq.slot[s] * keep * a.W + c;
-    float x[8], w[8];
-    ld8<float>(a.conv_b, c, acc);
-    for (int d = keep; d >= 0; --d) {  // d rows back
-      if (k - d >= 0) {
-        conv_input8<T>(a, m - d, c, bias, x);
-      } else if (start > 0) {
-        ld8<T>(a.state, st0 + (int64_t)(keep + k - d) * a.W, x);
-      } else {
-        continue;
-      }
-      ld8<float>(a.conv, (int64_t)(keep - d) * a.W + c, w);
-#pragma unroll
-      for (int j = 0; j < 8; ++j) acc[j] = fmaf(x[j], w[j], acc[j]);
-    }
-    st8<T>(a.u, (int64_t)m * a.W + c, acc);
-    if (m < a.singles && keep > 0) {
-      // x holds the row's own input: shift the state by one
-      float o[8];
-      for (int j = 0; j + 1 < keep; ++j) {
-        if (start > 0) {
-          ld8<T>(a.state, st0 + (int64_t)(j + 1) * a.W, o);
-        } else {
-#pragma unroll
-          for (int e = 0; e < 8; ++e) o[e] = 0.f;
-        }
-        st8<T>(a.state, st0 + (int64_t)j * a.W, o);
-      }
-      st8<T>(a.state, st0 + (int64_t)(keep - 1) * a.W, x);
-    }
-  }
-}
-
-// the last taps - 1 inputs of a sequence with n rows in this step, one channel per thread (ascending: what is read lies
-// ahead of what is written)
-template <typename T>
-__device__ __forceinline__ void conv_state_update(const RglruConv& a, int s, int c) {
-  const int n = a.seq.rows[s], start = a.seq.start[s], keep = a.taps - 1;
-  const int64_t st0 = (int64_t)a.seq.slot[s] * keep * a.W + c;
-  for (int j = 0; j < keep; ++j) {
-    const int k = n - keep + j;
-    float v = 0.f;
-    if (k >= 0)
-      v = source1<T>(a.src, a.seq.row0[s] + k, c) + a.bx[c];
-    else if (start > 0)
-      v = ld<T>(a.state, st0 + (int64_t)(n + j) * a.W);
-    st<T>(a.state, st0 + (int64_t)j * a.W, v);
+    for (int j = 0; j < 8; ++j)
+      acc[j] = sizeof(typename Raw<T>::type) == 4 ? gelu_tanh(acc[j] + bias[j]) : gelu_tanh_fast(acc[j] + bias[j]);
+    st8<T>(a.y, (int64_t)m * a.W + c, acc);
   }
 }
 
@@ -475,7 +375,7 @@ static int check_conv(const RglruConv& a, int src_f32, int splits, int64_t part_
                       const char* what) {
   SGLK_CHECK(a.M >= 0 && a.W > 0 && a.W % 8 == 0 && a.taps >= 1 && n_seqs >= 0 && a.singles >= 0 && a.singles <= a.M,
              "%s: bad shape", what);
-  SGLK_CHECK(a.M == 0 || (a.src.p && a.bx && a.by && a.conv && a.conv_b && a.u && a.y && a.seq.row_seq && a.seq.row0 && a.seq.rows &&
+  SGLK_CHECK(a.M == 0 || (a.src.p && a.bias && a.by && a.conv && a.conv_b && a.u && a.y && a.seq.row_seq && a.seq.row0 && a.seq.rows &&
                           a.seq.start && a.seq.slot && (a.state || a.taps == 1)),
              "%s: null pointer", what);
   SGLK_CHECK(aligned16(a.u) && aligned16(a.y) && aligned16(a.state), "%s: rows must be 16-byte aligned", what);
@@ -487,8 +387,11 @@ static int check_conv(const RglruConv& a, int src_f32, int splits, int64_t part_
       const float *conv, const float *conv_b, void *u, void *y, void *conv_state, const int32_t *row_seq, const int32_t *row0, \
       const int32_t *rows, const int32_t *start, const int32_t *slot, int M, int W, int taps, int singles, int n_seqs
 #define SGLK_CONV_MAKE                                                                                                \
-  RglruConv a { RowSource{src, src_f32, splits, part_stride, src_stride}, bx, by, conv, conv_b, u, y, conv_state,      \
-                RecurrentSeqs{row_seq, row0, rows, start, slot}, M, W, taps, singles }
+  RglruConv a {                                                                                                       \
+    ShortConv{RowSource{src, src_f32, splits, part_stride, src_stride}, bx, conv, conv_b, u, conv_state,              \
+              RecurrentSeqs{row_seq, row0, rows, start, slot}, M, W, taps, singles},                                  \
+        by, y                                                                                                         \
+  }
 
 extern "C" {
 

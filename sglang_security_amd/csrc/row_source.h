@@ -77,11 +77,18 @@ __device__ __forceinline__ float gelu_tanh_fast(float z) {
   return z * (1.0f - __builtin_amdgcn_rcpf(1.0f + __expf(2.0f * t)));
 }
 
+__device__ __forceinline__ float sigmoidf(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+
+__device__ __forceinline__ float silu_fast(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
+
+// 0 none, 1 square of relu, 2 gelu (tanh form), 3 silu
 __device__ __forceinline__ float activate(float z, int act) {
   if (act == 1) {
     const float r = fmaxf(z, 0.f);
     return r * r;
   }
+  if (act == 3) return z / (1.0f + expf(-z));
   return act == 2 ? gelu_tanh(z) : z;
 }
 

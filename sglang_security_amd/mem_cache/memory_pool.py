@@ -206,13 +206,27 @@ class MLATokenToKVPool:
         self.set_kv_buffer(layer, loc, row, row)
 
 
-class RecurrentStatePool:
-    """State of one recurrent layer: per slot the fp32 recurrence state and the last taps - 1 inputs of its convolution.
-    A slot is the request's row of the ReqToTokenPool.  Slots need no clearing: the kernels take the state as zero for a
-    sequence whose first row stands at position 0."""
+class TiedKVPool:
+    """Pool of attention whose values are its keys before their norm: per slot one row of all key/value heads and, in fp32,
+    the reciprocal root mean square of the row (the key norm's factor)."""
 
-    def __init__(self, slots: int, width: int, taps: int, dtype: torch.dtype, device: str):
-        self.state = torch.zeros((slots, width), dtype=torch.float32, device=device)
+    def __init__(self, size: int, row: int, dtype: torch.dtype, device: str):
+        self.size = size
+        self.rows = torch.zeros((size + 1, row), dtype=dtype, device=device)      # slot 0: dummy, as in the other pools
+        self.rms = torch.zeros(size + 1, dtype=torch.float32, device=device)
+
+    def get_size_bytes(self):
+        return sum(t.numel() * t.element_size() for t in (self.rows, self.rms))
+
+
+class RecurrentStatePool:
+    """State of one recurrent layer: per slot the fp32 recurrence state and the last taps - 1 inputs of its convolution over
+    `width` channels.  A slot is the request's row of the ReqToTokenPool.  Slots need no clearing: the kernels take the
+    state as zero for a sequence whose first row stands at position 0."""
+
+    def __init__(self, slots: int, width: int, taps: int, dtype: torch.dtype, device: str, state_shape=None):
+        """state_shape: of one slot's state (default: one number per channel)."""
+        self.state = torch.zeros((slots, *(state_shape or (width,))), dtype=torch.float32, device=device)
         self.conv = torch.zeros((slots, taps - 1, width), dtype=dtype, device=device)
 
     def get_size_bytes(self):
@@ -221,21 +235,38 @@ class RecurrentStatePool:
 
 class HybridCache:
     """What the layers of a decoder with mixed mixers keep between steps: one request table and one slot allocator for
-    all attention layers, a latent pool per attention layer and a state pool per recurrent layer (a layer that runs
-    several times has one of its own for every run).
+    all attention layers, a pool per attention layer and a state pool per recurrent layer (a layer that runs several times
+    has one of its own for every run).
 
-    layers: per layer run ("latent", latent, rotated part) or ("recurrent", width, taps).  The allocator's free list
-    lives on the host, where the engine lays its steps out."""
+    layers: per layer run
+        ("latent", latent, rotated part)       rows of latent attention
+        ("tied", elements of a row)            rows of tied attention
+        ("recurrent", width, taps)             one state per channel
+        ("matrix", width, taps, state shape)   states of any shape beside a convolution over `width` channels
+        ("parallel", [...])                    a tuple of the pools of mixers that stand side by side
+    The allocator's free list lives on the host, where the engine lays its steps out."""
 
     def __init__(self, layers, max_tokens: int, max_requests: int, max_context: int, dtype: torch.dtype, device):
         self.req_pool = ReqToTokenPool(max_requests, max_context, device)
-        self.layers = []
-        for kind, a, b in layers:
-            if kind == "latent":
-                self.layers.append(MLATokenToKVPool(max_tokens, 1, dtype, a, b, 1, device))
-            else:
-                self.layers.append(RecurrentStatePool(max_requests, a, b, dtype, device))
+        self._args = (max_tokens, max_requests, dtype, device)
+        self.layers = [self._pool(*spec) for spec in layers]
         self.allocator = TokenToKVPoolAllocator(max_tokens, dtype, "cpu", self)
 
+    def _pool(self, kind, *sizes):
+        max_tokens, max_requests, dtype, device = self._args
+        if kind == "latent":
+            return MLATokenToKVPool(max_tokens, 1, dtype, *sizes, 1, device)
+        if kind == "tied":
+            return TiedKVPool(max_tokens, *sizes, dtype, device)
+        if kind == "recurrent":
+            return RecurrentStatePool(max_requests, *sizes, dtype, device)
+        if kind == "matrix":
+            width, taps, shape = sizes
+            return RecurrentStatePool(max_requests, width, taps, dtype, device, shape)
+        if kind == "parallel":
+            return tuple(self._pool(*spec) for spec in sizes[0])
+        raise ValueError(f"unknown kind of cache {kind!r}")
+
     def get_size_bytes(self):
-        return sum(p.get_kv_size_bytes() if isinstance(p, MLATokenToKVPool) else p.get_size_bytes() for p in self.layers)
+        flat = [p for layer in self.layers for p in (layer if isinstance(layer, tuple) else (layer,))]
+        return sum(p.get_kv_size_bytes() if isinstance(p, MLATokenToKVPool) else p.get_size_bytes() for p in flat)

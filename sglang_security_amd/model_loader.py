@@ -9,7 +9,7 @@ import json
 import mmap
 import os
 import struct
-from typing import Dict, Tuple
+from typing import Dict, Optional, Tuple
 
 import torch
 
@@ -57,12 +57,13 @@ class Weights:
     def __contains__(self, name):
         return name in self._tensors
 
-    def get(self, name: str, shape: Tuple[int, ...], dtype: torch.dtype = None) -> torch.Tensor:
+    def get(self, name: str, shape: Tuple[Optional[int], ...], dtype: torch.dtype = None) -> torch.Tensor:
+        """shape: None where the tensor itself gives the size."""
         if name not in self._tensors:
             raise ValueError(f"the checkpoint has no tensor {name}")
         t = self._tensors[name]
         t = t() if callable(t) else t
-        if tuple(t.shape) != tuple(shape):
+        if len(t.shape) != len(shape) or any(want is not None and n != want for n, want in zip(t.shape, shape)):
             raise ValueError(f"{name}: shape {tuple(t.shape)}, the configuration asks for {tuple(shape)}")
         self.used.add(name)
         return t.to(device=self.device, dtype=dtype or self.dtype)

@@ -10,6 +10,15 @@ import importlib
 
 ARCHITECTURES = {
     "Lusatar": ("sglang_security_amd.models.lusatar", "Lusatar"),
+    "Kazedra": ("sglang_security_amd.models.kazedra", "Kazedra"),
+}
+
+# the kernel sources an architecture's steps launch beside those of every engine-served model
+COMMON_SOURCES = ("core.hip", "gemm_dense.hip", "residual_norm.hip")
+SAMPLING_SOURCES = ("elementwise.hip", "sampling.hip")
+SOURCES = {
+    "Lusatar": ("latent_attention.hip", "rglru.hip"),
+    "Kazedra": ("tied_attention.hip", "delta_rule.hip"),
 }
 
 SYNTHETIC = {
@@ -34,6 +43,12 @@ def model_class(config: dict):
         raise ValueError(f"unknown architecture {name!r}; known: {', '.join(sorted(ARCHITECTURES))}")
     module, cls = ARCHITECTURES[name]
     return getattr(importlib.import_module(module), cls)
+
+
+def kernel_sources(config: dict):
+    """What a checkout without a built library has to compile to step this model."""
+    model_class(config)
+    return COMMON_SOURCES + SOURCES[architecture_of(config)]
 
 
 def synthetic_config(name: str, *args):

@@ -18,8 +18,7 @@ from ..layers.latent_attention import LatentAttention
 from ..layers.linear import Linear, pad, padded, vector
 from ..layers.rglru import Rglru
 from ..layers.rotary import rotary_table
-
-LOGIT_ROWS = 64   # rows of the output product at a time: its split sums are vocab-wide
+from .output import output_logits
 
 
 @dataclasses.dataclass
@@ -192,8 +191,4 @@ class Lusatar:
         if W == 0:
             return None
         norm(**pending, h=h, w_next=self.final_norm, rows=batch.logit_rows, store_x=False)
-        logits = torch.empty(W, self.vocab, dtype=torch.float32, device=dev)
-        for i in range(0, W, LOGIT_ROWS):
-            out = logits[i: i + LOGIT_ROWS]
-            hops.capped_logits(self.head.source(h[i: i + out.shape[0]]), out, self.logit_cap, self.dtype)
-        return logits
+        return output_logits(self.head, h, W, self.vocab, self.logit_cap)

@@ -1,5 +1,5 @@
-"""Entry points over the C ABI for decoders with an fp32 residual stream, latent attention and gated linear recurrences:
-argument checks and launches on torch's current stream, in the manner of ops.py.
+"""Entry points over the C ABI for decoders with an fp32 residual stream, latent or tied attention, gated linear recurrences
+or delta rules: argument checks and launches on torch's current stream, in the manner of ops.py.
 
 A `Source` is a product's result on its way to the kernel that consumes it: fp32 split sums that nobody has added up yet,
 or finished rows of the activation type.
@@ -14,7 +14,7 @@ import torch
 from ._lib import SglkError, check, dtype_code, lib
 from .ops import _need_gpu, _ptr, _stream
 
-ACT_NONE, ACT_RELU2, ACT_GELU_TANH = 0, 1, 2
+ACT_NONE, ACT_RELU2, ACT_GELU_TANH, ACT_SILU = 0, 1, 2, 3
 
 
 @dataclasses.dataclass
@@ -37,6 +37,10 @@ class Source:
         if self.f32:
             return _ptr(d), 1, d.shape[0], d.stride(0), d.stride(1)
         return _ptr(d), 0, 1, 0, d.stride(0)
+
+    def columns(self, lo: int, hi: int) -> "Source":
+        """The same rows, columns [lo, hi) only (lo a multiple of eight)."""
+        return Source(self.data[..., lo:hi], self.f32)
 
 
 _NO_SOURCE = (0, 0, 1, 0, 0)
@@ -91,6 +95,15 @@ def source_act(src: Source, out, act, bias=None):
     _f32(bias, N, "source_act: bias")
     check(lib().sglk_source_act(*src.args(), _ptr(bias), _ptr(out), M, N, out.stride(0), int(act), dtype_code(out.dtype),
                                 _stream(out)), "source_act")
+    return out
+
+
+def source_gated_act(src: Source, out, act):
+    """out = act(first half of src's columns) * second half."""
+    M, N = out.shape
+    _src_ok(src, M, 2 * N, out.dtype, "source_gated_act")
+    check(lib().sglk_source_gated_act(*src.args(), _ptr(out), M, N, out.stride(0), int(act), dtype_code(out.dtype), _stream(out)),
+          "source_gated_act")
     return out
 
 
@@ -343,3 +356,172 @@ def rglru_rows(src, u, y, w, conv_state, state, seqs, out):
     check(lib().sglk_rglru_rows(*_conv_args(src, w, u, y, conv_state, seqs, 0), _ptr(w.wr), _ptr(w.wi), _ptr(w.br), _ptr(w.bi),
                                 _ptr(w.sp), _ptr(da), _ptr(db), _ptr(state), _ptr(out), out.stride(0), w.bwp, w.blocks,
                                 dtype_code(u.dtype), _stream(u)), "rglru_rows")
+
+
+# -------------------------------------------------------------------------------------------------- tied attention
+@dataclasses.dataclass
+class TiedWeights:
+    """What tied attention adds to the products of its queries and rows (everything in the base-2 domain)."""
+    bias: torch.Tensor       # [H, nb] by distance
+    sink: torch.Tensor       # [H]
+    heads: int
+    kv_heads: int
+    D: int                   # padded head size
+
+
+def tied_prep(src: Source, bias, wq, factor, q, pool, rms, loc, positions, q_size, k_size, eps):
+    """src [rows, q_cols + k_cols] -> q [rows, q_cols]; key rows to pool [slots, k_cols], their norms' factors to rms."""
+    M, q_cols = q.shape
+    k_cols = pool.shape[1]
+    _src_ok(src, M, q_cols + k_cols, q.dtype, "tied_prep")
+    _f32(bias, q_cols + k_cols, "tied_prep: bias")
+    _f32(wq, q_cols, "tied_prep: wq")
+    _f32(factor, 1, "tied_prep: factor")
+    _f32(rms, pool.shape[0], "tied_prep: rms")
+    _i32(loc, M, "tied_prep: loc")
+    _i32(positions, M, "tied_prep: positions")
+    if pool.dtype != q.dtype or pool.stride(1) != 1 or not q.is_contiguous():
+        raise SglkError("tied_prep: queries and pool rows do not match")
+    check(lib().sglk_tied_prep(*src.args(), _ptr(bias), _ptr(wq), _ptr(factor), _ptr(q), _ptr(pool), pool.stride(0), _ptr(rms),
+                               _ptr(loc), _ptr(positions), M, q_cols, k_cols, q_size, k_size, float(eps), dtype_code(q.dtype),
+                               _stream(q)), "tied_prep")
+
+
+def tied_supported(D) -> bool:
+    return bool(lib().sglk_tied_supported(D))
+
+
+def _tied_args(q, pool, rms, req_to_token, w: TiedWeights, what):
+    _need_gpu(q, pool, rms, req_to_token)
+    if q.dtype != pool.dtype or not q.is_contiguous() or q.shape[1] != w.heads * w.D or pool.stride(1) != 1 or \
+            pool.shape[1] < w.kv_heads * w.D or w.heads % w.kv_heads:
+        raise SglkError(f"{what}: query and pool rows do not match")
+    _f32(rms, pool.shape[0], f"{what}: rms")
+    _f32(w.bias, w.heads, f"{what}: bias")
+    _f32(w.sink, w.heads, f"{what}: sink")
+    if req_to_token.dtype != torch.int32 or w.bias.shape[0] != w.heads:
+        raise SglkError(f"{what}: request table or bias table do not match")
+    return (_ptr(q), _ptr(pool), pool.stride(0), _ptr(rms), _ptr(req_to_token), req_to_token.stride(0), _ptr(w.bias),
+            w.bias.shape[1], _ptr(w.sink), w.heads, w.kv_heads, w.D)
+
+
+def _tied_out(out, q, w, what):
+    if out.shape != (q.shape[0], w.heads * w.D) or out.dtype != q.dtype or out.stride(1) != 1:
+        raise SglkError(f"{what}: out must be [rows, heads * D]")
+
+
+def tied_decode(q, pool, rms, req_to_token, req, positions, w: TiedWeights, part, lse):
+    """q [M, H * D], every row a request's last one -> part [M, H, S, D], lse [M, H, S]."""
+    M, S = q.shape[0], lse.shape[2]
+    if q.dtype != torch.bfloat16:
+        raise SglkError("tied_decode: bf16 only")
+    args = _tied_args(q, pool, rms, req_to_token, w, "tied_decode")
+    _i32(req, M, "tied_decode: req")
+    _i32(positions, M, "tied_decode: positions")
+    _f32(part, M * w.heads * S * w.D, "tied_decode: part")
+    _f32(lse, M * w.heads * S, "tied_decode: lse")
+    check(lib().sglk_tied_decode(*args, _ptr(req), _ptr(positions), _ptr(part), _ptr(lse), M, S, _stream(q)), "tied_decode")
+
+
+def tied_merge(part, lse, w: TiedWeights, out, out_scale=1.0):
+    M, H, S, D = part.shape
+    _f32(part, M * H * S * D, "tied_merge: part")
+    _f32(lse, M * H * S, "tied_merge: lse")
+    if out.shape != (M, H * D) or out.stride(1) != 1 or (H, D) != (w.heads, w.D):
+        raise SglkError("tied_merge: out must be [rows, heads * D]")
+    check(lib().sglk_tied_merge(_ptr(part), _ptr(lse), _ptr(w.sink), S, float(out_scale), _ptr(out), out.stride(0), M, H, D,
+                                dtype_code(out.dtype), _stream(out)), "tied_merge")
+
+
+def tied_prefill(q, pool, rms, req_to_token, row0, rows, start, req, max_rows, w: TiedWeights, out, out_scale=1.0):
+    """Runs of rows (row0, rows, position of the first row, request per sequence); q, out: all rows of the step."""
+    n = rows.numel()
+    if q.dtype != torch.bfloat16:
+        raise SglkError("tied_prefill: bf16 only")
+    args = _tied_args(q, pool, rms, req_to_token, w, "tied_prefill")
+    _tied_out(out, q, w, "tied_prefill")
+    for t in (row0, rows, start, req):
+        _i32(t, n, "tied_prefill: sequence arrays")
+    check(lib().sglk_tied_prefill(*args, _ptr(row0), _ptr(rows), _ptr(start), _ptr(req), n, int(max_rows), float(out_scale),
+                                  _ptr(out), out.stride(0), _stream(q)), "tied_prefill")
+
+
+def tied_rows(q, pool, rms, req_to_token, req, positions, w: TiedWeights, out, out_scale=1.0):
+    """Every row of q by itself: any size and float type."""
+    M = q.shape[0]
+    args = _tied_args(q, pool, rms, req_to_token, w, "tied_rows")
+    _tied_out(out, q, w, "tied_rows")
+    _i32(req, M, "tied_rows: req")
+    _i32(positions, M, "tied_rows: positions")
+    check(lib().sglk_tied_rows(*args, _ptr(req), _ptr(positions), float(out_scale), _ptr(out), out.stride(0), M,
+                               dtype_code(q.dtype), _stream(q)), "tied_rows")
+
+
+# ------------------------------------------------------------------------------------------------ gated delta rule
+def short_conv(src: Source, conv, u, conv_state, seqs: RowSeqs, singles, act=ACT_NONE, bias=None, conv_b=None):
+    """u [rows, W] = act(convolution); conv [taps, W]; conv_state [slots, taps - 1, W]."""
+    M, W = u.shape
+    taps, n = conv.shape[0], seqs.rows.numel()
+    _src_ok(src, M, W, u.dtype, "short_conv")
+    _f32(conv, taps * W, "short_conv: conv")
+    _f32(bias, W, "short_conv: bias")
+    _f32(conv_b, W, "short_conv: conv_b")
+    _i32(seqs.row_seq, M, "short_conv: row_seq")
+    for t in (seqs.row0, seqs.rows, seqs.start, seqs.slot):
+        _i32(t, n, "short_conv: sequence arrays")
+    if conv.shape[1] != W or not u.is_contiguous():
+        raise SglkError("short_conv: filters or rows do not match")
+    if conv_state.shape[1:] != (taps - 1, W) or conv_state.dtype != u.dtype or not conv_state.is_contiguous():
+        raise SglkError("short_conv: convolution state does not match")
+    check(lib().sglk_short_conv(*src.args(), _ptr(bias), _ptr(conv), _ptr(conv_b), _ptr(u), _ptr(conv_state), _ptr(seqs.row_seq),
+                                _ptr(seqs.row0), _ptr(seqs.rows), _ptr(seqs.start), _ptr(seqs.slot), M, W, taps, int(singles), n,
+                                int(act), dtype_code(u.dtype), _stream(u)), "short_conv")
+
+
+@dataclasses.dataclass
+class DeltaWeights:
+    """One gated delta mixer's parameters and sizes in the kernels' layout."""
+    rate: torch.Tensor       # [heads] exp(A_log)
+    dt: torch.Tensor         # [heads]
+    norm: torch.Tensor       # [vp]
+    heads: int
+    kv_heads: int
+    dp: int                  # padded key and value sizes, then the true ones
+    vp: int
+    dim: int
+    vdim: int
+    b_col: int               # columns of the step sizes and decays behind the gates
+    a_col: int
+    eps: float
+
+    @property
+    def channels(self):
+        return 2 * self.kv_heads * self.dp + self.heads * self.vp
+
+
+def _delta_args(u, src: Source, w: DeltaWeights, state, seqs: RowSeqs, out, out_scale, what):
+    M = u.shape[0]
+    _src_ok(src, M, w.a_col + w.heads, u.dtype, what)
+    _f32(w.rate, w.heads, f"{what}: rate")
+    _f32(w.dt, w.heads, f"{what}: dt")
+    _f32(w.norm, w.vp, f"{what}: norm")
+    _f32(state, 0, f"{what}: state")
+    n = seqs.rows.numel()
+    _i32(seqs.row_seq, M, f"{what}: row_seq")
+    for t in (seqs.row0, seqs.rows, seqs.start, seqs.slot):
+        _i32(t, n, f"{what}: sequence arrays")
+    if u.shape[1] != w.channels or u.stride(1) != 1 or state.shape[1:] != (w.heads, w.dp, w.vp):
+        raise SglkError(f"{what}: channels or state do not match")
+    if out.shape != (M, w.heads * w.vp) or out.dtype != u.dtype or out.stride(1) != 1:
+        raise SglkError(f"{what}: out must be [rows, heads * vp]")
+    return (_ptr(u), u.stride(0), *src.args(), w.b_col, w.a_col, _ptr(w.rate), _ptr(w.dt), _ptr(w.norm), _ptr(state), _ptr(out),
+            out.stride(0), _ptr(seqs.row_seq), _ptr(seqs.row0), _ptr(seqs.rows), _ptr(seqs.start), _ptr(seqs.slot), M, w.kv_heads,
+            w.heads, w.dp, w.vp, w.dim, w.vdim, float(out_scale), float(w.eps))
+
+
+def delta_step(u, src, w: DeltaWeights, state, seqs, out, out_scale, seq0, n_seqs):
+    """Sequences seq0 .. n_seqs - 1, row after row; u, src, out: all rows of the step."""
+    if n_seqs > seqs.rows.numel():
+        raise SglkError("delta_step: sequence range")
+    check(lib().sglk_delta_step(*_delta_args(u, src, w, state, seqs, out, out_scale, "delta_step"), int(seq0), int(n_seqs),
+                                dtype_code(u.dtype), _stream(u)), "delta_step")

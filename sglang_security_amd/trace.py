@@ -31,11 +31,14 @@ def main(argv=None) -> int:
 
     import torch
 
+    from . import build
     from .engine import Engine, Entry
-    from .models import load_model
+    from .model_loader import load_config
+    from .models import kernel_sources, load_model
 
     if not torch.cuda.is_available():
         raise RuntimeError("no GPU (there is no CPU fallback)")
+    build.ensure(kernel_sources(load_config(args.model)))
     torch.backends.cuda.matmul.allow_tf32 = False
     torch.backends.cuda.matmul.allow_bf16_reduced_precision_reduction = False
     dev = torch.device("cuda", 0)

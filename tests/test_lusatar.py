@@ -261,11 +261,13 @@ def test_scheduler_portions_admission_and_reuse():
 
 
 def test_a_partial_library_is_enough_for_the_engine_only(monkeypatch, tmp_path):
-    from sglang_security_amd import _lib, build
+    from sglang_security_amd import _lib, build, models
 
     monkeypatch.setattr(_lib, "_lib", None)
     monkeypatch.setattr(_lib, "_partial", True)
     lib = _lib.lib()
     assert lib.sglk_residual_norm(*([None] * 2 + [None, 0, 1.0, None, 0, 1, 0, 0, None, None, 0, None, None, None, 0, None, 0, 1, 8, 8,
                                                   1e-5, 2, None])) == -1
-    assert set(build.ENGINE) <= {p.split("/")[-1] for p in build._sources()}
+    here = {p.split("/")[-1] for p in build._sources()}
+    for name in models.ARCHITECTURES:
+        assert set(models.kernel_sources({"architecture": name}) + models.SAMPLING_SOURCES) <= here
