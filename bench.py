@@ -37,13 +37,14 @@ def parse():
     ap.add_argument("--suffix", type=int, default=128)
     ap.add_argument("--quant", default="awq", choices=["awq", "bf16", "fp8"])
     ap.add_argument("--model", default="llama3-8b", choices=["llama3-8b", "llama3-70b-tp8-rank", "qwen2-0.5b", "deepseek-v3-dense",
-                                                             "lusatar-2b", "lusatar-8b"],
+                                                             "lusatar-2b", "lusatar-8b", "kazedra-2b", "kazedra-8b"],
                     help="llama3-70b-tp8-rank: one rank's shard of Llama-3-70B under TP=8 (no all-reduce on one GPU); "
                          "qwen2-0.5b: the reference's CPU-runnable plumbing case, use with --quant bf16 --batch 1 "
                          "--prefix 0 --suffix 128 (head size 64: the generic attention kernels); deepseek-v3-dense: "
                          "the three dense layers of DeepSeek-V3 (absorbed MLA over a latent KV pool + block-fp8 "
                          "projections), a layer-stack workload, not a whole model; lusatar-2b / lusatar-8b: latent attention and gated "
-                         "linear recurrences through the engine (decode and prefill, bf16)")
+                         "linear recurrences through the engine (decode and prefill, bf16); kazedra-2b / kazedra-8b: attention and a gated "
+                         "delta rule side by side, likewise")
     ap.add_argument("--tp", action="store_true",
                     help="the ranks form ONE tensor-parallel group (use with --model llama3-70b-tp8-rank --gpus 8): "
                          "peer-to-peer all-reduce after o / down, value = tokens/s of the one sharded model")
@@ -499,13 +500,13 @@ def main():
     from sglang_security_amd.benchlib import aggregate
     from sglang_security_amd.decode_runner import LlamaConfig, LlamaDecoder
 
-    if args.model == "deepseek-v3-dense" or args.model.startswith("lusatar"):
+    if args.model == "deepseek-v3-dense" or args.model.startswith(("lusatar", "kazedra")):
         if args.model == "deepseek-v3-dense":
             out = deepseek_dense_workload(args, dev, world)
         else:
-            from sglang_security_amd.benchlib_engine import lusatar_workload
+            from sglang_security_amd.benchlib_engine import engine_workload
 
-            out = lusatar_workload(args, dev, world)
+            out = engine_workload(args, dev, world)
         if rank == 0:
             print(json.dumps(out), flush=True)
         if world > 1:

@@ -1145,6 +1145,18 @@ SGLK_API int sglk_delta_step(const void* u, int64_t u_stride, const void* src, i
                              const int32_t* row0, const int32_t* rows, const int32_t* start, const int32_t* slot, int M,
                              int kv_heads, int heads, int dp, int vp, int dim, int vdim, float out_scale, float eps,
                              int seq0, int n_seqs, int dtype, void* stream);
+/* bf16: the same for the rows from first_row on, in tiles of 64 rows of a sequence (tile_row, tile_rows; tile0 per
+ * sequence: its first tile); o [M][heads * vp] fp32 scratch */
+SGLK_API int sglk_delta_chunk_supported(int dp, int vp);
+SGLK_API int64_t sglk_delta_chunk_workspace_bytes(int tiles, int heads);
+SGLK_API int sglk_delta_chunk(const void* u, int64_t u_stride, const void* src, int src_f32, int splits, int64_t part_stride,
+                              int64_t src_stride, int b_col, int a_col, const float* rate, const float* dt,
+                              const float* norm, float* state, void* out, int64_t out_stride, const int32_t* row_seq,
+                              const int32_t* row0, const int32_t* rows, const int32_t* start, const int32_t* slot, int M,
+                              int kv_heads, int heads, int dp, int vp, int dim, int vdim, float out_scale, float eps,
+                              const int32_t* tile_row, const int32_t* tile_rows, const int32_t* tile0, int tiles,
+                              void* workspace, int64_t workspace_bytes, float* o, int first_row, int seq0, int n_seqs,
+                              void* stream);
 
 #ifdef __cplusplus
 }

@@ -166,6 +166,10 @@ _SIGS = {
     "sglk_short_conv": (i32, [p, i32, i32, i64, i64] + [p] * 10 + [i32] * 7 + [p]),
     "sglk_delta_step": (i32, [p, i64, p, i32, i32, i64, i64, i32, i32, p, p, p, p, p, i64] + [p] * 5 + [i32] * 7 +
                         [f32, f32, i32, i32, i32, p]),
+    "sglk_delta_chunk_supported": (i32, [i32, i32]),
+    "sglk_delta_chunk_workspace_bytes": (i64, [i32, i32]),
+    "sglk_delta_chunk": (i32, [p, i64, p, i32, i32, i64, i64, i32, i32, p, p, p, p, p, i64] + [p] * 5 + [i32] * 7 +
+                         [f32, f32, p, p, p, i32, p, i64, p, i32, i32, i32, p]),
     "sglk_ar_meta_size": (i64, []),
     "sglk_ar_init": (i64, [p, i32, i32, i32, i64]),
     "sglk_ar_init_handles": (i64, [p, p, i64, p, p, i32, i32, i32, i64]),

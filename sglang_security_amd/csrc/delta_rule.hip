@@ -8,11 +8,25 @@
 //   short_conv     convolution and activation of the q, k and v channels; the states of the convolution
 //   delta_step     one sequence and head per block, row after row, the state in registers: single rows, and
 //                  portions of any type and size
+//   delta_prep     portions in tiles of 64 rows, one wave per tile and head: what the tile's rows do to each other
+//   delta_chunk    walks the tiles of a sequence: the state in registers, every product on the matrix cores
+//   delta_gate     norm and gate of the rows delta_chunk leaves
 //
-// The state is read once per row: o = g S^T q + (k . q) u needs the products of the old state only.  The unit norms stay
-// factors on the products of the convolution's outputs, so they are never rounded to the activation type.
+// delta_step reads the state once per row: o = g S^T q + (k . q) u needs the products of the old state only.  The unit
+// norms stay factors on the products of the convolution's outputs, so they are never rounded to the activation type.
+//
+// A tile of rows 1 .. n in front of which the state is S0, with c_i the product of its first i decays:
+//
+//   u_i = beta_i (v_i - c_i S0^T k_i) - sum_{j < i} A_ij u_j,     A_ij = beta_i (k_i . k_j) c_i / c_j
+//   o_i = c_i S0^T q_i + sum_{j <= i} P_ij u_j,                   P_ij = (q_i . k_j) c_i / c_j
+//   S   = c_n S0 + sum_j (c_n / c_j) k_j u_j^T
+//
+// so U = T (beta V - beta c K S0) with T = (1 + A)^-1, which does not depend on the state.  The convolution's outputs enter
+// the matrix cores as the 16-bit numbers they are; every other operand (T, P, states, u) as the sum of two bfloat16
+// numbers, which leaves 2^-17 of it, and products are added in fp32.
 #include <algorithm>
 
+#include "attention_tile.h"
 #include "common.h"
 #include "row_source.h"
 #include "short_conv.h"
@@ -201,6 +215,430 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaRule a, int seq0) 
   }
 }
 
+// ---------------------------------------------------------------------------------------------------------------------
+// tiles of 64 rows
+// ---------------------------------------------------------------------------------------------------------------------
+constexpr int kDeltaTile = 64;
+constexpr int kDeltaFrag = 4 * 2 * 2 * 64 * 8;  // a 64 x 64 matrix as operands: [row block][k-step of 32][high, low][lane][8]
+
+// what delta_prep leaves per (tile, head)
+struct DeltaTiles {
+  uint16_t* mats;   // [tiles][VH][T, P][kDeltaFrag]
+  float* rows;      // [tiles][VH][64][4]: beta, beta c / |k|, c / |q|, (c_n / c) / |k|   (|q| with the query's scale)
+  float* decay;     // [tiles][VH]: c_n
+};
+
+__device__ __forceinline__ void split_bf16(float x, uint16_t& hi, uint16_t& lo) {
+  hi = Conv<bf16_t>::from_f32(x);
+  lo = Conv<bf16_t>::from_f32(x - Conv<bf16_t>::to_f32(hi));
+}
+
+__device__ __forceinline__ void split4(const float4v& x, short4v& hi, short4v& lo) {
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    uint16_t a, b;
+    split_bf16(x[r], a, b);
+    hi[r] = (short)a;
+    lo[r] = (short)b;
+  }
+}
+
+__device__ __forceinline__ void wave_lds_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+}
+
+constexpr int kMatPitch = 68;  // floats
+constexpr int kDeltaPrepLds = 4 * (64 * kMatPitch + 4 * 64) * 4;
+
+// the lower triangle of a wave's 64 x 64 matrix in LDS -> operands: lane (i, g) of step s holds the columns
+// 32 s + (j < 4 ? 4 g + j : 16 + 4 g + j - 4) of row i, the order transposed LDS reads deliver a tile's rows in
+__device__ __forceinline__ void store_operands(const float* mat, uint16_t* __restrict__ out) {
+  const int lane = threadIdx.x & 63, i16 = lane & 15, g = lane >> 4;
+#pragma unroll
+  for (int rb = 0; rb < 4; ++rb)
+#pragma unroll
+    for (int s = 0; s <= rb / 2; ++s) {
+      const float* row = mat + (16 * rb + i16) * kMatPitch + 32 * s + 4 * g;
+      short4v h0, l0, h1, l1;
+      split4(*reinterpret_cast<const float4v*>(row), h0, l0);
+      split4(*reinterpret_cast<const float4v*>(row + 16), h1, l1);
+      uint16_t* o = out + ((rb * 2 + s) * 2 * 64 + lane) * 8;
+      *reinterpret_cast<short8*>(o) = short8{h0[0], h0[1], h0[2], h0[3], h1[0], h1[1], h1[2], h1[3]};
+      *reinterpret_cast<short8*>(o + 64 * 8) = short8{l0[0], l0[1], l0[2], l0[3], l1[0], l1[1], l1[2], l1[3]};
+    }
+}
+
+// One wave per (tile, head).
+__global__ void __launch_bounds__(256, 2) delta_prep_kernel(DeltaRule a, DeltaTiles t, const int32_t* __restrict__ tile_row,
+                                                            const int32_t* __restrict__ tile_rows) {
+  extern __shared__ __attribute__((aligned(16))) float prep_lds[];
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int i16 = lane & 15, g = lane >> 4;
+  const int h = blockIdx.x * 4 + wid, tile = blockIdx.y;
+  if (h >= a.VH) return;  // wave-uniform; no block barrier below
+  float* mat = prep_lds + wid * (64 * kMatPitch + 4 * 64);
+  float* rk = mat + 64 * kMatPitch;
+  float* rq = rk + 64;
+  float* cum = rq + 64;   // log2 of the running decay
+  float* bet = cum + 64;
+  const int row0 = tile_row[tile], valid = tile_rows[tile];
+  float log_g, beta;
+  delta_gates<bf16_t>(a, row0 + min(lane, valid - 1), h, log_g, beta);
+  float c = lane < valid ? log_g * 1.4426950408889634f : 0.f;
+  if (lane >= valid) beta = 0.f;
+#pragma unroll
+  for (int o = 1; o < 64; o <<= 1) {
+    const float up = __shfl_up(c, o, 64);
+    if (lane >= o) c += up;
+  }
+  cum[lane] = c;
+  bet[lane] = beta;
+
+  const int kh = h / (a.VH / a.KH);
+  const uint16_t* u = reinterpret_cast<const uint16_t*>(a.u) + kh * a.dp + 8 * g;
+  const uint16_t* qrow[4];
+#pragma unroll
+  for (int rb = 0; rb < 4; ++rb) qrow[rb] = u + (int64_t)(row0 + min(16 * rb + i16, valid - 1)) * a.u_stride;
+  const int koff = a.KH * a.dp;
+  float4v G[10], P[10];  // tiles (bi, bj), bj <= bi, at bi (bi + 1) / 2 + bj
+#pragma unroll
+  for (int i = 0; i < 10; ++i) G[i] = P[i] = float4v{0.f, 0.f, 0.f, 0.f};
+  float sk[4] = {0.f, 0.f, 0.f, 0.f}, sq[4] = {0.f, 0.f, 0.f, 0.f};
+  for (int ks = 0; ks < a.dp / 32; ++ks) {
+    short8 kf[4], qf[4];
+#pragma unroll
+    for (int rb = 0; rb < 4; ++rb) {
+      qf[rb] = *reinterpret_cast<const short8*>(qrow[rb] + 32 * ks);
+      kf[rb] = *reinterpret_cast<const short8*>(qrow[rb] + koff + 32 * ks);
+    }
+#pragma unroll
+    for (int rb = 0; rb < 4; ++rb) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const float kv = Conv<bf16_t>::to_f32((uint16_t)kf[rb][j]), qv = Conv<bf16_t>::to_f32((uint16_t)qf[rb][j]);
+        sk[rb] = fmaf(kv, kv, sk[rb]);
+        sq[rb] = fmaf(qv, qv, sq[rb]);
+      }
+#pragma unroll
+      for (int bj = 0; bj <= rb; ++bj) {
+        G[rb * (rb + 1) / 2 + bj] = Mfma16<bf16_t>::mma(kf[rb], kf[bj], G[rb * (rb + 1) / 2 + bj]);
+        P[rb * (rb + 1) / 2 + bj] = Mfma16<bf16_t>::mma(qf[rb], kf[bj], P[rb * (rb + 1) / 2 + bj]);
+      }
+    }
+  }
+#pragma unroll
+  for (int rb = 0; rb < 4; ++rb) {
+    float x = sk[rb], y = sq[rb];
+    x += __shfl_xor(x, 16, 64);
+    x += __shfl_xor(x, 32, 64);
+    y += __shfl_xor(y, 16, 64);
+    y += __shfl_xor(y, 32, 64);
+    if (g == 0) {
+      rk[16 * rb + i16] = 1.0f / sqrtf(x + kUnitEps);
+      rq[16 * rb + i16] = a.q_scale / sqrtf(y + kUnitEps);
+    }
+  }
+  wave_lds_sync();
+  const int64_t th = (int64_t)tile * a.VH + h;
+  const float total = cum[63], e = __builtin_amdgcn_exp2f(c);
+  *reinterpret_cast<float4v*>(t.rows + (th * 64 + lane) * 4) =
+      float4v{beta, beta * e * rk[lane], e * rq[lane], __builtin_amdgcn_exp2f(total - c) * rk[lane]};
+  if (lane == 0) t.decay[th] = __builtin_amdgcn_exp2f(total);
+
+  // both matrices pass through the wave's LDS: P, then A and its triangular inverse
+  uint16_t* out = t.mats + th * 2 * kDeltaFrag;
+#pragma unroll
+  for (int which = 1; which >= 0; --which) {
+#pragma unroll
+    for (int bi = 0; bi < 4; ++bi)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = 16 * bi + 4 * g + r;
+        const float ci = cum[i], left = which ? rq[i] : bet[i] * rk[i];
+#pragma unroll
+        for (int bj = 0; bj < 4; ++bj) {
+          const int j = 16 * bj + i16;
+          float v = 0.f;
+          if (bj <= bi && (which ? j <= i : j < i))
+            v = (which ? P : G)[bi * (bi + 1) / 2 + (bj <= bi ? bj : 0)][r] * left * rk[j] * __builtin_amdgcn_exp2f(ci - cum[j]);
+          mat[i * kMatPitch + j] = v;
+        }
+      }
+    wave_lds_sync();
+    if (which == 0) {
+      // lane j owns column j of T: t_i = [i == j] - sum_{l < i} A_il t_l
+      float tc[64];
+#pragma unroll
+      for (int i = 0; i < 64; ++i) {
+        float s[4] = {i == lane ? 1.f : 0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int l = 0; l < i; l += 4) {
+          const float4v row = *reinterpret_cast<const float4v*>(mat + i * kMatPitch + l);  // columns from i on are zero
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            if (l + j < i) s[j] = fmaf(-row[j], tc[l + j], s[j]);
+        }
+        tc[i] = (s[0] + s[1]) + (s[2] + s[3]);
+      }
+      wave_lds_sync();
+#pragma unroll
+      for (int i = 0; i < 64; ++i) mat[i * kMatPitch + lane] = tc[i];
+      wave_lds_sync();
+    }
+    store_operands(mat, out + which * kDeltaFrag);
+    wave_lds_sync();
+  }
+}
+
+constexpr int delta_x_pitch(int DP) { return DP * 2 + 16; }
+constexpr int delta_r_pitch(int NT) { return NT * 32 + 16; }
+constexpr int delta_st_bytes(int DP, int NT) {
+  const int st = 2 * NT * 16 * delta_x_pitch(DP), u = 2 * 64 * delta_r_pitch(NT);
+  return st > u ? st : u;
+}
+constexpr int delta_chunk_lds(int DP, int NT) {
+  return delta_st_bytes(DP, NT) + 64 * delta_x_pitch(DP) + 2 * 64 * delta_r_pitch(NT);
+}
+
+// 16 columns of 32 rows (32 step ..) of a row-major 16-bit tile, as an operand: lane (i, g) gets column 16 block + i of the rows
+// (j < 4 ? 4 g + j : 16 + 4 g + j - 4)
+__device__ __forceinline__ short8 read_columns(const char* tile, int pitch, int step, int block) {
+  const int lane = threadIdx.x & 63, hl = lane & 15, g = lane >> 4;
+  const char* p = tile + (32 * step + 4 * g + (hl >> 2)) * pitch + 32 * block + 8 * (hl & 3);
+  const short4v lo = lds_read_tr16(p), hi = lds_read_tr16(p + 16 * pitch);
+  return short8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+}
+
+// Block: one sequence, one head, 16 NT columns of its values.  Wave w owns the rows 16 w .. of every tile (as columns of
+// the products) and the state's rows 16 w .., 16 (w + 4) .. in accumulators.  o: [rows, VH * vp] fp32 before norm and gate.
+template <int DP, int NT>
+__global__ void __launch_bounds__(256, delta_chunk_lds(DP, NT) <= 80 * 1024 ? 2 : 1)
+    delta_chunk_kernel(DeltaRule a, DeltaTiles t, const int32_t* __restrict__ tile0, float* __restrict__ o, int seq0) {
+  constexpr int KS = DP / 32, KB = (DP + 63) / 64, XP = delta_x_pitch(DP), RP = delta_r_pitch(NT);
+  extern __shared__ __attribute__((aligned(16))) char dc_lds[];
+  char* st_hi = dc_lds;                       // S^T [16 NT][DP], then u [64][16 NT]
+  char* st_lo = st_hi + NT * 16 * XP;
+  char* u_hi = dc_lds;
+  char* u_lo = u_hi + 64 * RP;
+  char* xk = dc_lds + delta_st_bytes(DP, NT);  // k [64][DP]
+  char* r_hi = xk + 64 * XP;                  // the right-hand side [64][16 NT], then u c_n / c
+  char* r_lo = r_hi + 64 * RP;
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int i16 = lane & 15, g = lane >> 4;
+  const int h = blockIdx.x, n0 = blockIdx.y * 16 * NT, s = seq0 + blockIdx.z;
+  const int nt_used = min(NT, (a.vp - n0) / 16);
+  const int row0 = a.seq.row0[s], n = a.seq.rows[s];
+  const int tiles = (n + kDeltaTile - 1) / kDeltaTile;
+  const int64_t first = tile0[s];
+  const int kh = h / (a.VH / a.KH);
+  float* state = a.state + ((int64_t)a.seq.slot[s] * a.VH + h) * a.dp * a.vp + n0 + i16;
+  const bool fresh = a.seq.start[s] == 0;
+  float4v S[KB][NT];
+#pragma unroll
+  for (int i = 0; i < KB; ++i)
+#pragma unroll
+    for (int nt = 0; nt < NT; ++nt) {
+      S[i][nt] = float4v{0.f, 0.f, 0.f, 0.f};
+      const int kb = wid + 4 * i;
+      if (!fresh && 16 * kb < DP && nt < nt_used) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) S[i][nt][r] = state[(int64_t)(16 * kb + 4 * g + r) * a.vp + 16 * nt];
+      }
+    }
+  const uint16_t* u = reinterpret_cast<const uint16_t*>(a.u);
+  short8 kf[KS], qf[KS], tf[2][2], pf[2][2];
+  short4v vf[NT];
+  float4v sc;
+  float dec;
+  auto row_of = [&](int tile) { return (int64_t)(row0 + min(64 * tile + 16 * wid + i16, n - 1)); };
+  auto fetch_x = [&](int tile) {
+    const uint16_t* p = u + row_of(tile) * a.u_stride + kh * a.dp + 8 * g;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      qf[ks] = *reinterpret_cast<const short8*>(p + 32 * ks);
+      kf[ks] = *reinterpret_cast<const short8*>(p + a.KH * a.dp + 32 * ks);
+    }
+  };
+  auto fetch_v = [&](int tile) {
+    const uint16_t* p = u + row_of(tile) * a.u_stride + 2 * a.KH * a.dp + h * a.vp + n0 + 4 * g;
+#pragma unroll
+    for (int nt = 0; nt < NT; ++nt) vf[nt] = nt < nt_used ? *reinterpret_cast<const short4v*>(p + 16 * nt) : short4v{0, 0, 0, 0};
+  };
+  auto fetch_mat = [&](short8(&f)[2][2], int tile, int which) {
+    const uint16_t* p = t.mats + (((first + tile) * a.VH + h) * 2 + which) * kDeltaFrag + wid * 4 * 512 + 8 * lane;
+#pragma unroll
+    for (int st = 0; st < 2; ++st)
+      if (st <= wid / 2) {
+#pragma unroll
+        for (int hl = 0; hl < 2; ++hl) f[st][hl] = *reinterpret_cast<const short8*>(p + (st * 2 + hl) * 512);
+      }
+  };
+  auto fetch_rows = [&](int tile) {
+    const int64_t th = (first + tile) * a.VH + h;
+    sc = *reinterpret_cast<const float4v*>(t.rows + (th * 64 + 16 * wid + i16) * 4);
+    dec = t.decay[th];
+  };
+  fetch_x(0);
+  fetch_v(0);
+  fetch_rows(0);
+  fetch_mat(tf, 0, 0);
+  fetch_mat(pf, 0, 1);
+  for (int tile = 0; tile < tiles; ++tile) {
+    const int next = min(tile + 1, tiles - 1);
+    // the state in front of the tile, two 16-bit halves, transposed; the tile's keys
+#pragma unroll
+    for (int i = 0; i < KB; ++i) {
+      const int kb = wid + 4 * i;
+      if (16 * kb < DP) {
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt) {
+          short4v hi, lo;
+          split4(S[i][nt], hi, lo);
+          *reinterpret_cast<short4v*>(st_hi + (16 * nt + i16) * XP + (16 * kb + 4 * g) * 2) = hi;
+          *reinterpret_cast<short4v*>(st_lo + (16 * nt + i16) * XP + (16 * kb + 4 * g) * 2) = lo;
+        }
+      }
+    }
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) *reinterpret_cast<short8*>(xk + (16 * wid + i16) * XP + (4 * ks + g) * 16) = kf[ks];
+    __syncthreads();
+    float4v oacc[NT];
+#pragma unroll
+    for (int nt = 0; nt < NT; ++nt) {
+      float4v y = float4v{0.f, 0.f, 0.f, 0.f}, z = y;
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        const short8 hi = *reinterpret_cast<const short8*>(st_hi + (16 * nt + i16) * XP + (4 * ks + g) * 16);
+        const short8 lo = *reinterpret_cast<const short8*>(st_lo + (16 * nt + i16) * XP + (4 * ks + g) * 16);
+        y = Mfma16<bf16_t>::mma(hi, kf[ks], y);
+        z = Mfma16<bf16_t>::mma(hi, qf[ks], z);
+        y = Mfma16<bf16_t>::mma(lo, kf[ks], y);
+        z = Mfma16<bf16_t>::mma(lo, qf[ks], z);
+      }
+      float4v r;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) r[e] = sc[0] * Conv<bf16_t>::to_f32((uint16_t)vf[nt][e]) - sc[1] * y[e];
+      short4v hi, lo;
+      split4(r, hi, lo);
+      *reinterpret_cast<short4v*>(r_hi + (16 * wid + i16) * RP + (16 * nt + 4 * g) * 2) = hi;
+      *reinterpret_cast<short4v*>(r_lo + (16 * wid + i16) * RP + (16 * nt + 4 * g) * 2) = lo;
+      oacc[nt] = z * sc[2];
+    }
+    const float tail = sc[3], d = dec;
+    fetch_x(next);  // the next tile's operands fly during the rest of this one
+    fetch_v(next);
+    fetch_rows(next);
+    __syncthreads();
+    float4v uacc[NT];
+#pragma unroll
+    for (int nt = 0; nt < NT; ++nt) uacc[nt] = float4v{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int st = 0; st < 2; ++st)
+      if (st <= wid / 2) {  // wave-uniform: T is lower triangular
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt) {
+          const short8 hi = read_columns(r_hi, RP, st, nt), lo = read_columns(r_lo, RP, st, nt);
+          uacc[nt] = Mfma16<bf16_t>::mma(hi, tf[st][0], uacc[nt]);
+          uacc[nt] = Mfma16<bf16_t>::mma(lo, tf[st][0], uacc[nt]);
+          uacc[nt] = Mfma16<bf16_t>::mma(hi, tf[st][1], uacc[nt]);
+        }
+      }
+    fetch_mat(tf, next, 0);
+    __syncthreads();  // the right-hand side and the state's copy have been read
+#pragma unroll
+    for (int nt = 0; nt < NT; ++nt) {
+      const int at = (16 * wid + i16) * RP + (16 * nt + 4 * g) * 2;
+      short4v hi, lo;
+      split4(uacc[nt], hi, lo);
+      *reinterpret_cast<short4v*>(u_hi + at) = hi;
+      *reinterpret_cast<short4v*>(u_lo + at) = lo;
+      split4(uacc[nt] * tail, hi, lo);
+      *reinterpret_cast<short4v*>(r_hi + at) = hi;
+      *reinterpret_cast<short4v*>(r_lo + at) = lo;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int st = 0; st < 2; ++st)
+      if (st <= wid / 2) {
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt) {
+          const short8 hi = read_columns(u_hi, RP, st, nt), lo = read_columns(u_lo, RP, st, nt);
+          oacc[nt] = Mfma16<bf16_t>::mma(hi, pf[st][0], oacc[nt]);
+          oacc[nt] = Mfma16<bf16_t>::mma(lo, pf[st][0], oacc[nt]);
+          oacc[nt] = Mfma16<bf16_t>::mma(hi, pf[st][1], oacc[nt]);
+        }
+      }
+    fetch_mat(pf, next, 1);
+    const int i = 64 * tile + 16 * wid + i16;
+    if (i < n) {
+      float* dst = o + (int64_t)(row0 + i) * (a.VH * a.vp) + h * a.vp + n0 + 4 * g;
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt)
+        if (nt < nt_used) *reinterpret_cast<float4v*>(dst + 16 * nt) = oacc[nt];
+    }
+#pragma unroll
+    for (int k = 0; k < KB; ++k)
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt) S[k][nt] *= d;
+#pragma unroll
+    for (int st = 0; st < 2; ++st) {
+      short8 kc[KB];
+#pragma unroll
+      for (int k = 0; k < KB; ++k) kc[k] = read_columns(xk, XP, st, min(wid + 4 * k, DP / 16 - 1));
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt) {
+        const short8 hi = read_columns(r_hi, RP, st, nt), lo = read_columns(r_lo, RP, st, nt);
+#pragma unroll
+        for (int k = 0; k < KB; ++k) {
+          S[k][nt] = Mfma16<bf16_t>::mma(kc[k], hi, S[k][nt]);
+          S[k][nt] = Mfma16<bf16_t>::mma(kc[k], lo, S[k][nt]);
+        }
+      }
+    }
+    __syncthreads();  // keys and u have been read
+  }
+#pragma unroll
+  for (int i = 0; i < KB; ++i) {
+    const int kb = wid + 4 * i;
+    if (16 * kb < DP) {
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt)
+        if (nt < nt_used) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) state[(int64_t)(16 * kb + 4 * g + r) * a.vp + 16 * nt] = S[i][nt][r];
+        }
+    }
+  }
+}
+
+// norm over a head's values, its weight and gate: TPH threads per (row, head), eight values each
+template <typename T>
+__global__ void __launch_bounds__(256) delta_gate_kernel(DeltaRule a, const float* __restrict__ o, int M0, int M, int TPH) {
+  const int64_t idx = ((int64_t)blockIdx.x * 256 + threadIdx.x) / TPH;
+  const int t = threadIdx.x & (TPH - 1), c = 8 * t;
+  const bool live = idx < (int64_t)(M - M0) * a.VH && c < a.vp;
+  const int64_t mh = live ? idx : 0;
+  const int m = M0 + (int)(mh / a.VH), h = (int)(mh % a.VH);
+  float v[8], w[8], z[8], ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v[j] = 0.f;
+  if (live) {
+    ld8<float>(o, (int64_t)m * (a.VH * a.vp) + h * a.vp + c, v);
+    ld8<float>(a.norm, c, w);
+    source8<T>(a.src, m, h * a.vp + c, z);
+  }
+#pragma unroll
+  for (int j = 0; j < 8; ++j) ss += v[j] * v[j];
+  for (int off = 1; off < TPH; off <<= 1) ss += __shfl_xor(ss, off, 64);
+  if (!live) return;
+  const float inv = a.out_scale / sqrtf(ss / (float)a.vdim + a.eps);
+#pragma unroll
+  for (int j = 0; j < 8; ++j)
+    v[j] *= inv * w[j] * (sizeof(typename Raw<T>::type) == 2 ? silu_fast(z[j]) : activate(z[j], 3));
+  st8<T>(a.out, (int64_t)m * a.out_stride + h * a.vp + c, v);
+}
+
 }  // namespace sglk
 
 using namespace sglk;
@@ -288,6 +726,67 @@ int sglk_delta_step(SGLK_DELTA_ARGS, int seq0, int n_seqs, int dtype, void* stre
       SGLK_DS(0);
   });
 #undef SGLK_DS
+  SGLK_LAUNCH_CHECK();
+  return SGLK_OK;
+}
+
+// head sizes delta_chunk has tile kernels for
+#define SGLK_DELTA_SIZES(X) X(32) X(64) X(96) X(128) X(192) X(256)
+
+int sglk_delta_chunk_supported(int dp, int vp) {
+  if (vp % 16 != 0 || vp <= 0 || vp > 512) return 0;
+#define X(S) if (dp == S) return 1;
+  SGLK_DELTA_SIZES(X)
+#undef X
+  return 0;
+}
+
+// bytes of delta_chunk's workspace for that many tiles
+int64_t sglk_delta_chunk_workspace_bytes(int tiles, int heads) {
+  return (int64_t)tiles * heads * (2 * kDeltaFrag * 2 + 64 * 16 + 4) + 16;
+}
+
+int sglk_delta_chunk(SGLK_DELTA_ARGS, const int32_t* tile_row, const int32_t* tile_rows, const int32_t* tile0, int tiles,
+                     void* workspace, int64_t workspace_bytes, float* o, int first_row, int seq0, int n_seqs, void* stream) {
+  SGLK_DELTA_MAKE;
+  if (int rc = check_delta(a, M, dim, seq0, n_seqs, SGLK_BF16, "delta_chunk")) return rc;
+  SGLK_CHECK(sglk_delta_chunk_supported(dp, vp), "delta_chunk: no tile kernel for heads of %d / %d", dp, vp);
+  SGLK_CHECK(tiles >= 0 && tiles <= 65535 && first_row >= 0 && first_row <= M, "delta_chunk: bad shape");
+  if (M == first_row || n_seqs == seq0 || tiles == 0) return SGLK_OK;
+  SGLK_CHECK(tile_row && tile_rows && tile0 && workspace && o && aligned16(workspace) && aligned16(o),
+             "delta_chunk: null or unaligned pointer");
+  SGLK_CHECK(workspace_bytes >= sglk_delta_chunk_workspace_bytes(tiles, heads), "delta_chunk: workspace too small");
+  DeltaTiles t;
+  t.mats = (uint16_t*)workspace;
+  t.rows = (float*)(t.mats + (int64_t)tiles * heads * 2 * kDeltaFrag);
+  t.decay = t.rows + (int64_t)tiles * heads * 64 * 4;
+  hipStream_t s = (hipStream_t)stream;
+  if (int rc = ensure_lds<delta_prep_kernel>(kDeltaPrepLds)) return rc;
+  hipLaunchKernelGGL(delta_prep_kernel, dim3((heads + 3) / 4, tiles), dim3(256), kDeltaPrepLds, s, a, t, tile_row, tile_rows);
+  SGLK_LAUNCH_CHECK();
+  // 64 columns of values per block, 32 where that leaves half of the chip idle
+  const int wide = vp > 32 && (int64_t)heads * (n_seqs - seq0) * ((vp + 63) / 64) >= 192;
+#define SGLK_DC(S, NT)                                                                                                   \
+  {                                                                                                                      \
+    if (int rc = ensure_lds<delta_chunk_kernel<S, NT>>(delta_chunk_lds(S, NT))) return rc;                               \
+    hipLaunchKernelGGL((delta_chunk_kernel<S, NT>), dim3(heads, (vp + 16 * NT - 1) / (16 * NT), n_seqs - seq0), dim3(256), \
+                       delta_chunk_lds(S, NT), s, a, t, tile0, o, seq0);                                                 \
+  }
+#define X(S)         \
+  if (dp == S) {     \
+    if (wide)        \
+      SGLK_DC(S, 4)  \
+    else             \
+      SGLK_DC(S, 2)  \
+  }
+  SGLK_DELTA_SIZES(X)
+#undef X
+#undef SGLK_DC
+  SGLK_LAUNCH_CHECK();
+  int tph = 1;
+  while (tph * 8 < vp) tph *= 2;
+  const int64_t threads = (int64_t)(M - first_row) * heads * tph;
+  hipLaunchKernelGGL((delta_gate_kernel<bf16_t>), dim3((unsigned)((threads + 255) / 256)), dim3(256), 0, s, a, o, first_row, M, tph);
   SGLK_LAUNCH_CHECK();
   return SGLK_OK;
 }

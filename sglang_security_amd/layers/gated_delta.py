@@ -1,7 +1,8 @@
 """Gated delta rule: heads with a matrix state that is decayed, corrected towards the current value along the current key,
 and read by the query; short convolutions with silu in front, a gated norm per head behind.
 
-Key and value sizes are padded to multiples of 32 and 16 (zeros).  The mixer owns rows of a stacked input product (`w_in`)
+Rows that are a sequence's only row of the step are walked one by one, longer portions in tiles of 64 rows; types or sizes
+without a tile kernel are walked row after row.  Key and value sizes are padded to multiples of 32 and 16 (zeros).  The mixer owns rows of a stacked input product (`w_in`)
 and columns of a stacked output product (`w_out`): see layers/parallel.py.
 """
 from __future__ import annotations
@@ -23,6 +24,7 @@ class GatedDelta:
             raise ValueError(f"{H} heads over {K} query/key heads")
         dp, vp, Hp = pad(dim, 32), pad(vdim, 16), pad(H, 8)
         self.dtype, self.out_scale, self.taps = dtype, out_scale, c["conv"]
+        self.tiles = dtype == torch.bfloat16 and hops.delta_chunk_supported(dp, vp)
         f32 = lambda name: weight(name, torch.float32)
 
         def heads(t, n, d, to):
@@ -50,4 +52,9 @@ class GatedDelta:
         u = torch.empty(T, w.channels, dtype=self.dtype, device=out.device)
         hops.short_conv(src.columns(0, w.channels), self.conv, u, pool.conv, seqs, n1, hops.ACT_SILU)
         gates = src.columns(w.channels, src.cols)
-        hops.delta_step(u, gates, w, pool.state, seqs, out, self.out_scale, 0, seqs.rows.numel())
+        n = seqs.rows.numel()
+        step_to = n1 if self.tiles else n                # sequences that are walked row after row
+        if step_to:
+            hops.delta_step(u, gates, w, pool.state, seqs, out, self.out_scale, 0, step_to)
+        if step_to < n:
+            hops.delta_chunk(u, gates, w, pool.state, seqs, out, self.out_scale, n1, n1, batch.tile_row, batch.tile_rows, batch.tile0)

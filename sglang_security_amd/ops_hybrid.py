@@ -525,3 +525,22 @@ def delta_step(u, src, w: DeltaWeights, state, seqs, out, out_scale, seq0, n_seq
         raise SglkError("delta_step: sequence range")
     check(lib().sglk_delta_step(*_delta_args(u, src, w, state, seqs, out, out_scale, "delta_step"), int(seq0), int(n_seqs),
                                 dtype_code(u.dtype), _stream(u)), "delta_step")
+
+
+def delta_chunk_supported(dp, vp) -> bool:
+    return bool(lib().sglk_delta_chunk_supported(dp, vp))
+
+
+def delta_chunk(u, src, w: DeltaWeights, state, seqs, out, out_scale, first_row, seq0, tile_row, tile_rows, tile0):
+    """Rows from first_row on (sequences from seq0 on), in tiles of 64 rows of one sequence."""
+    M, tiles, n = u.shape[0], tile_row.numel(), seqs.rows.numel()
+    if u.dtype != torch.bfloat16:
+        raise SglkError("delta_chunk: bf16 only")
+    _i32(tile_row, tiles, "delta_chunk: tile_row")
+    _i32(tile_rows, tiles, "delta_chunk: tile_rows")
+    _i32(tile0, n, "delta_chunk: tile0")
+    size = lib().sglk_delta_chunk_workspace_bytes(tiles, w.heads)
+    ws = torch.empty(size, dtype=torch.uint8, device=u.device)
+    o = torch.empty(M, w.heads * w.vp, dtype=torch.float32, device=u.device)
+    check(lib().sglk_delta_chunk(*_delta_args(u, src, w, state, seqs, out, out_scale, "delta_chunk"), _ptr(tile_row), _ptr(tile_rows),
+                                 _ptr(tile0), tiles, _ptr(ws), size, _ptr(o), int(first_row), int(seq0), n, _stream(u)), "delta_chunk")
