@@ -1109,11 +1109,11 @@ SGLK_API int sglk_tied_prep(const void* src, int src_f32, int splits, int64_t pa
                             int k_cols, int q_size, int k_size, float eps, int dtype, void* stream);
 SGLK_API int sglk_tied_supported(int D);
 /* bf16 rows of one token each over positions [0, p] of request req[m]: normalised partials part [M][H][splits][D], lse
- * base 2 (-inf: empty split), without the sink */
+ * base 2 (-inf: empty split), without the sink; out (one split): finished rows instead */
 SGLK_API int sglk_tied_decode(const void* q, const void* pool, int64_t pool_stride, const float* rms,
                               const int32_t* req_to_token, int64_t r2t_stride, const float* bias, int nb, const float* sink,
                               int H, int kv_heads, int D, const int32_t* req, const int32_t* positions, float* part,
-                              float* lse, int M, int splits, void* stream);
+                              float* lse, int M, int splits, float out_scale, void* out, int64_t out_stride, void* stream);
 /* out[m][h * D ..] = out_scale * the merged partials, the sink counted */
 SGLK_API int sglk_tied_merge(const float* part, const float* lse, const float* sink, int splits, float out_scale, void* out,
                              int64_t out_stride, int M, int H, int D, int dtype, void* stream);

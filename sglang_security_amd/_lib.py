@@ -159,7 +159,7 @@ _SIGS = {
         i32, p, p, p, p, p, p, p, p, p, i64, i32, i32, i32, p]),
     "sglk_tied_prep": (i32, [p, i32, i32, i64, i64] + [p] * 5 + [i64] + [p] * 3 + [i32] * 5 + [f32, i32, p]),
     "sglk_tied_supported": (i32, [i32]),
-    "sglk_tied_decode": (i32, [p, p, i64, p, p, i64, p, i32, p, i32, i32, i32, p, p, p, p, i32, i32, p]),
+    "sglk_tied_decode": (i32, [p, p, i64, p, p, i64, p, i32, p, i32, i32, i32, p, p, p, p, i32, i32, f32, p, i64, p]),
     "sglk_tied_merge": (i32, [p, p, p, i32, f32, p, i64, i32, i32, i32, i32, p]),
     "sglk_tied_prefill": (i32, [p, p, i64, p, p, i64, p, i32, p, i32, i32, i32, p, p, p, p, i32, i32, f32, p, i64, p]),
     "sglk_tied_rows": (i32, [p, p, i64, p, p, i64, p, i32, p, i32, i32, i32, p, p, f32, p, i64, i32, i32, p]),

@@ -92,15 +92,15 @@ __device__ __forceinline__ void block_sum3(float& x, float& y, float& z, float* 
 __host__ __device__ inline int delta_step_lds(int dp, int vp) { return (2 * dp + 2 * (256 / (vp / 4)) * vp + vp) * 4; }
 
 // Block: one head of one sequence.  Thread (rg, cg) owns the columns 4 cg .. + 3 of the state's rows rg, rg + RG, ...; NR of
-// them per thread in registers (NR = 0: any number, the state stays in memory).
-template <typename T, int NR>
+// them per thread in registers (NR = 0: any number, the state stays in memory).  EXACT: every thread owns NR rows.
+template <typename T, int NR, bool EXACT>
 __global__ void __launch_bounds__(256) delta_step_kernel(DeltaRule a, int seq0) {
   extern __shared__ __attribute__((aligned(16))) float delta_lds[];
   __shared__ float red3[12], red1[4];
   const int h = blockIdx.x, s = seq0 + blockIdx.y;
   const int CG = a.vp / 4, RG = 256 / CG;
   const int cg = threadIdx.x % CG, rg = threadIdx.x / CG;
-  const bool mine = rg < RG;
+  const bool mine = EXACT || rg < RG;
   float* kx = delta_lds;            // [dp] key channels, then [dp] query channels
   float* qx = kx + a.dp;
   float* part = qx + a.dp;          // [2][RG][vp]
@@ -110,12 +110,15 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaRule a, int seq0) 
   float* sp = a.state + ((int64_t)a.seq.slot[s] * a.VH + h) * a.dp * a.vp + 4 * cg;
   const int kh = h / (a.VH / a.KH);
   const float4v zero = float4v{0.f, 0.f, 0.f, 0.f};
+  float* base = sp + (int64_t)rg * a.vp;
   float4v S[NR > 0 ? NR : 1];
   if constexpr (NR > 0) {
 #pragma unroll
     for (int i = 0; i < NR; ++i) {
       const int r = rg + RG * i;
-      S[i] = mine && r < a.dp && !fresh ? *reinterpret_cast<const float4v*>(sp + (int64_t)r * a.vp) : zero;
+      S[i] = zero;  // states are read and written once: past the caches
+      if (!fresh && mine && (EXACT || r < a.dp))
+        S[i] = __builtin_nontemporal_load(reinterpret_cast<const float4v*>(base + (int64_t)(RG * i) * a.vp));
     }
   } else if (fresh && mine) {
     for (int r = rg; r < a.dp; r += RG) *reinterpret_cast<float4v*>(sp + (int64_t)r * a.vp) = zero;
@@ -143,7 +146,7 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaRule a, int seq0) 
       if constexpr (NR > 0) {
 #pragma unroll
         for (int i = 0; i < NR; ++i) {
-          const int r = min(rg + RG * i, a.dp - 1);  // rows past the state are zero
+          const int r = EXACT ? rg + RG * i : min(rg + RG * i, a.dp - 1);  // rows past the state are zero
           ak += S[i] * kx[r];
           aq += S[i] * qx[r];
         }
@@ -186,7 +189,7 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaRule a, int seq0) 
 #pragma unroll
         for (int i = 0; i < NR; ++i) {
           const int r = rg + RG * i;
-          if (r < a.dp) S[i] = S[i] * g + u * kx[r];
+          if (EXACT || r < a.dp) S[i] = S[i] * g + u * kx[r];
         }
       } else {
         for (int r = rg; r < a.dp; r += RG) {
@@ -210,7 +213,8 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaRule a, int seq0) 
 #pragma unroll
     for (int i = 0; i < NR; ++i) {
       const int r = rg + RG * i;
-      if (mine && r < a.dp) *reinterpret_cast<float4v*>(sp + (int64_t)r * a.vp) = S[i];
+      if (mine && (EXACT || r < a.dp))
+        __builtin_nontemporal_store(S[i], reinterpret_cast<float4v*>(base + (int64_t)(RG * i) * a.vp));
     }
   }
 }
@@ -712,18 +716,21 @@ int sglk_delta_step(SGLK_DELTA_ARGS, int seq0, int n_seqs, int dtype, void* stre
   const int RG = 256 / (vp / 4), per = (dp + RG - 1) / RG;
   const int lds = delta_step_lds(dp, vp);
   const dim3 grid(heads, n_seqs - seq0);
-#define SGLK_DS(NR) hipLaunchKernelGGL((delta_step_kernel<T, NR>), grid, dim3(256), lds, (hipStream_t)stream, a, seq0)
+  const bool exact = 256 % (vp / 4) == 0 && per * RG == dp;
+#define SGLK_DS(NR, E) hipLaunchKernelGGL((delta_step_kernel<T, NR, E>), grid, dim3(256), lds, (hipStream_t)stream, a, seq0)
   SGLK_DISPATCH_FLOAT(dtype, T, {
-    if (per <= 4)
-      SGLK_DS(4);
+    if (exact && per == 4)
+      SGLK_DS(4, true);
+    else if (exact && per == 8)
+      SGLK_DS(8, true);
+    else if (exact && per == 16)
+      SGLK_DS(16, true);
     else if (per <= 8)
-      SGLK_DS(8);
-    else if (per <= 16)
-      SGLK_DS(16);
+      SGLK_DS(8, false);
     else if (per <= 32)
-      SGLK_DS(32);
+      SGLK_DS(32, false);
     else
-      SGLK_DS(0);
+      SGLK_DS(0, false);
   });
 #undef SGLK_DS
   SGLK_LAUNCH_CHECK();

@@ -9,7 +9,8 @@
 // the query's weight, the bias table and the sinks).
 //
 //   tied_prep      the projections' rows -> queries; rows and reciprocal root mean squares into the pool
-//   tied_decode    single rows over the pool, split over the context, every wave with tiles of its own
+//   tied_decode    single rows over the pool, split over the context, every wave with tiles of its own; with one split
+//                  the rows are finished
 //   tied_merge     split partials and the sink -> output rows
 //   tied_prefill   runs of rows over the pool, 64 or 128 rows of a head per block
 //   tied_rows      one wave per (row, head): any size and type
@@ -117,6 +118,9 @@ struct TiedSplit {
   float* part;               // [M][H][splits][D]
   float* lse;                // [M][H][splits], base 2 (-inf: nothing in this split)
   int splits;
+  uint16_t* out;             // one split only: finished rows [M, out_stride], head h at h * D, instead of a partial
+  int64_t out_stride;
+  float out_scale;
 };
 
 __host__ __device__ constexpr int tied_decode_lds(int D) { return 4 * (kTile * tied_pitch(D) + kTile * 4); }
@@ -289,14 +293,26 @@ __global__ void __launch_bounds__(256, D <= 128 && HT == 1 ? 3 : 1) tied_decode_
       tot += w[i] * stat[1][u][i][c];
     }
     const int64_t o = ((int64_t)b * a.H + kv * a.share + sub) * s.splits + split;
-    const float inv = 1.0f / tot;
+    float inv = 1.0f / tot;
+    if (s.out) {  // the sink joins under the larger of the two maxima
+      const float sink = a.sink[kv * a.share + sub], both = fmaxf(top, sink), own = exp2f(top - both);
+      inv = s.out_scale * own / (tot * own + exp2f(sink - both));
+    }
     for (int d = 4 * e; d < D; d += 64) {
       float4v v = float4v{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int i = 0; i < 4; ++i) v += *reinterpret_cast<const float4v*>(obuf + (i * 16 + c) * OP + d) * w[i];
-      *reinterpret_cast<float4v*>(s.part + o * D + d) = v * inv;
+      v *= inv;
+      if (s.out) {
+        short4v pk;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) pk[i] = (short)Conv<bf16_t>::from_f32(v[i]);
+        *reinterpret_cast<short4v*>(s.out + b * s.out_stride + (kv * a.share + sub) * D + d) = pk;
+      } else {
+        *reinterpret_cast<float4v*>(s.part + o * D + d) = v;
+      }
     }
-    if (e == 0) s.lse[o] = top + log2f(tot);
+    if (e == 0 && !s.out) s.lse[o] = top + log2f(tot);
   }
 }
 
@@ -629,15 +645,18 @@ int sglk_tied_supported(int D) {
 }
 
 int sglk_tied_decode(SGLK_TIED_ARGS, const int32_t* req, const int32_t* positions, float* part, float* lse, int M, int splits,
-                     void* stream) {
+                     float out_scale, void* out, int64_t out_stride, void* stream) {
   SGLK_TIED_MAKE("tied_decode");
   if (int rc = check_tied(a, M, D, "tied_decode")) return rc;
   SGLK_CHECK(sglk_tied_supported(D), "tied_decode: no tile kernel for heads of %d", D);
   SGLK_CHECK(splits >= 1 && splits <= 65535, "tied_decode: bad split count");
   if (M == 0) return SGLK_OK;
-  SGLK_CHECK(req && positions && part && lse && aligned16(part) && aligned16(q) && aligned16(pool) && pool_stride % 8 == 0,
+  SGLK_CHECK(req && positions && (out || (part && lse)) && aligned16(part) && aligned16(q) && aligned16(pool) &&
+                 pool_stride % 8 == 0 && aligned16(out),
              "tied_decode: null or unaligned pointer");
-  const TiedSplit s{req, positions, part, lse, splits};
+  SGLK_CHECK(!out || (splits == 1 && out_stride >= (int64_t)H * D && out_stride % 8 == 0),
+             "tied_decode: finished rows come of one split");
+  const TiedSplit s{req, positions, part, lse, splits, (uint16_t*)out, out_stride, out_scale};
   const int ht = a.share > 16 && D <= 128 ? 2 : 1;
   const dim3 grid(M, kv_heads * ((a.share + 16 * ht - 1) / (16 * ht)), splits);
   SGLK_CHECK(grid.y <= 65535, "tied_decode: too many heads");

@@ -54,9 +54,9 @@ class TiedAttention:
         return ("tied", self.G * self.D)
 
     def _splits(self, rows: int, max_context: int) -> int:
-        """Splits of a row's context: enough blocks for four rounds of the chip, a tile for each of a block's waves."""
+        """Splits of a row's context: two blocks for every unit of the chip, a tile for each of a block's waves."""
         blocks = rows * self.G * ((self.H // self.G + 15) // 16)
-        return max(1, min(64, (1024 + blocks - 1) // blocks, (max_context + 127) // 128))
+        return max(1, min(64, (512 + blocks - 1) // blocks, (max_context + 127) // 128))
 
     def mix(self, src, batch, pool, out):
         """src: the rows' columns of the stacked input product; pool: the layer's TiedKVPool; out [rows, H * D]."""
@@ -70,6 +70,9 @@ class TiedAttention:
             return
         if n1:
             S = self._splits(n1, batch.max_context)
+        if n1 and S == 1:
+            hops.tied_decode(q[:n1], *kv, batch.row_req, batch.positions, self.w, out=out[:n1], out_scale=self.out_scale)
+        elif n1:
             part = torch.empty(n1, self.H, S, self.D, dtype=torch.float32, device=out.device)
             lse = torch.empty(n1, self.H, S, dtype=torch.float32, device=out.device)
             hops.tied_decode(q[:n1], *kv, batch.row_req, batch.positions, self.w, part, lse)

@@ -410,17 +410,24 @@ def _tied_out(out, q, w, what):
         raise SglkError(f"{what}: out must be [rows, heads * D]")
 
 
-def tied_decode(q, pool, rms, req_to_token, req, positions, w: TiedWeights, part, lse):
-    """q [M, H * D], every row a request's last one -> part [M, H, S, D], lse [M, H, S]."""
-    M, S = q.shape[0], lse.shape[2]
+def tied_decode(q, pool, rms, req_to_token, req, positions, w: TiedWeights, part=None, lse=None, out=None, out_scale=1.0):
+    """q [M, H * D], every row a request's last one -> part [M, H, S, D], lse [M, H, S]; or, unsplit, finished rows out."""
+    M = q.shape[0]
     if q.dtype != torch.bfloat16:
         raise SglkError("tied_decode: bf16 only")
     args = _tied_args(q, pool, rms, req_to_token, w, "tied_decode")
     _i32(req, M, "tied_decode: req")
     _i32(positions, M, "tied_decode: positions")
-    _f32(part, M * w.heads * S * w.D, "tied_decode: part")
-    _f32(lse, M * w.heads * S, "tied_decode: lse")
-    check(lib().sglk_tied_decode(*args, _ptr(req), _ptr(positions), _ptr(part), _ptr(lse), M, S, _stream(q)), "tied_decode")
+    S = 1
+    if out is not None:
+        _tied_out(out, q, w, "tied_decode")
+        part = lse = None
+    else:
+        S = lse.shape[2]
+        _f32(part, M * w.heads * S * w.D, "tied_decode: part")
+        _f32(lse, M * w.heads * S, "tied_decode: lse")
+    check(lib().sglk_tied_decode(*args, _ptr(req), _ptr(positions), _ptr(part), _ptr(lse), M, S, float(out_scale), _ptr(out),
+                                 0 if out is None else out.stride(0), _stream(q)), "tied_decode")
 
 
 def tied_merge(part, lse, w: TiedWeights, out, out_scale=1.0):

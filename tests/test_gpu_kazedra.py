@@ -120,6 +120,10 @@ def test_tied_decode(H_, G, D, dim, buckets, longest):
         H.tied_merge(part, lse, w, out[:, : H_ * D], 0.75)
         close(out[:, : H_ * D].view(n, H_, D), want, 1e-2, f"{S} splits")
         assert bool((out[:, H_ * D:] == 3.0).all())
+    out = torch.full((n, H_ * D + 8), 3.0, dtype=BF16, device=DEV)
+    H.tied_decode(q.view(n, -1).to(DEV), pd, *args, out=out[:, : H_ * D], out_scale=0.75)
+    close(out[:, : H_ * D].view(n, H_, D), want, 1e-2, "finished")
+    assert bool((out[:, H_ * D:] == 3.0).all())
     for dt, tol in ((BF16, 1e-2), (F32, 1e-5)):
         out = torch.empty(n, H_ * D, dtype=dt, device=DEV)
         H.tied_rows(q.view(n, -1).to(dt).to(DEV), pd.to(dt), *args, out, 0.75)
@@ -355,6 +359,11 @@ def test_token_by_token_equals_the_prompt(engines, name, dtype):
     e = engines(name, dtype)
     run(e, name, [{0: p} for p in cut(3, 150, [1])])                      # graph replays from the third step on
     run(e, name, [{0: p} for p in cut(4, 300, [180] + [1] * 120)])
+
+
+@pytest.mark.parametrize("name", list(K.CONFIGS))
+def test_contexts_too_short_to_split(engines, name):
+    run(engines(name, BF16, max_context=100), name, [{0: a, 1: b} for a, b in zip(cut(5, 90, [1]), cut(6, 97, [7] + [1] * 90))])
 
 
 @pytest.mark.parametrize("name,dtype", CASES)
