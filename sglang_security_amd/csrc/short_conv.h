@@ -83,6 +83,35 @@ __device__ __forceinline__ void short_conv_rows(const ShortConv& a, int m0, int 
       return;
     }
   }
+  if constexpr (R == 1) {
+    // four taps, a sequence's only row: the whole state and every filter on their way at once
+    if (keep == 3 && m0 < a.singles) {
+      const int s = a.seq.row_seq[m0];
+      const int64_t st0 = (int64_t)a.seq.slot[s] * 3 * a.W + c;
+      float x[4][8], w[4][8];
+      conv_input8<T>(a, m0, c, bias, x[3]);
+#pragma unroll
+      for (int t = 0; t < 4; ++t) ld8<float>(a.conv, (int64_t)t * a.W + c, w[t]);
+      ld8_or_zero(a.conv_b, c, acc);
+#pragma unroll
+      for (int j = 0; j < 3; ++j) ld8<T>(a.state, st0 + (int64_t)j * a.W, x[j]);
+      const bool fresh = a.seq.start[s] == 0;
+#pragma unroll
+      for (int j = 0; j < 3; ++j)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[j][e] = fresh ? 0.f : x[j][e];
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[e] = fmaf(x[t][e], w[t][e], acc[e]);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc[e] = conv_act<T, ACT>(acc[e]);
+      st8<T>(a.u, (int64_t)m0 * a.W + c, acc);
+#pragma unroll
+      for (int j = 0; j < 3; ++j) st8<T>(a.state, st0 + (int64_t)j * a.W, x[j + 1]);
+      return;
+    }
+  }
   for (int m = m0; m < min(m0 + R, a.M); ++m) {
     const int s = a.seq.row_seq[m];
     const int start = a.seq.start[s];

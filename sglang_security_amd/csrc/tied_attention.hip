@@ -44,18 +44,23 @@ struct TiedPrep {
   float eps;
 };
 
-template <typename T, int VPT>
-__global__ void __launch_bounds__(256) tied_prep_kernel(TiedPrep a) {
-  __shared__ float red[2][4];
+// one block of BT threads per row, VPT pieces of eight elements per thread
+template <typename T, int BT, int VPT>
+__global__ void __launch_bounds__(BT) tied_prep_kernel(TiedPrep a) {
+  constexpr int NW = BT / 64;
+  __shared__ float red[2][NW];
   const int m = blockIdx.x, vq = a.q_cols / 8, nv = vq + a.k_cols / 8;
-  float x[VPT][8], sq = 0.f, sk = 0.f;
+  const float factor = a.factor[a.positions[m]];
+  const int64_t slot = a.loc[m];
+  float x[VPT][8], w[VPT][8], sq = 0.f, sk = 0.f;
 #pragma unroll
   for (int i = 0; i < VPT; ++i) {
-    const int v = threadIdx.x + 256 * i;
+    const int v = threadIdx.x + BT * i;
     if (v >= nv) continue;
     float b[8];
     source8<T>(a.src, m, 8 * v, x[i]);
     ld8<float>(a.bias, 8 * v, b);
+    if (v < vq) ld8<float>(a.wq, 8 * v, w[i]);
     float ss = 0.f;
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
@@ -74,21 +79,22 @@ __global__ void __launch_bounds__(256) tied_prep_kernel(TiedPrep a) {
     red[1][threadIdx.x >> 6] = sk;
   }
   __syncthreads();
-  sq = red[0][0] + red[0][1] + red[0][2] + red[0][3];
-  sk = red[1][0] + red[1][1] + red[1][2] + red[1][3];
-  const float iq = a.factor[a.positions[m]] / sqrtf(sq / (float)a.q_size + a.eps);
-  const int64_t slot = a.loc[m];
+  sq = sk = 0.f;
+#pragma unroll
+  for (int i = 0; i < NW; ++i) {
+    sq += red[0][i];
+    sk += red[1][i];
+  }
+  const float iq = factor / sqrtf(sq / (float)a.q_size + a.eps);
   if (threadIdx.x == 0) a.rms[slot] = 1.0f / sqrtf(sk / (float)a.k_size + a.eps);
 #pragma unroll
   for (int i = 0; i < VPT; ++i) {
-    const int v = threadIdx.x + 256 * i;
+    const int v = threadIdx.x + BT * i;
     if (v >= nv) continue;
     if (v < vq) {
-      float w[8];
-      ld8<float>(a.wq, 8 * v, w);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) w[j] *= x[i][j] * iq;
-      st8<T>(a.q, (int64_t)m * a.q_cols + 8 * v, w);
+      for (int j = 0; j < 8; ++j) w[i][j] *= x[i][j] * iq;
+      st8<T>(a.q, (int64_t)m * a.q_cols + 8 * v, w[i]);
     } else {
       st8<T>(a.pool, slot * a.pool_stride + 8 * (v - vq), x[i]);
     }
@@ -621,15 +627,20 @@ int sglk_tied_prep(const void* src, int src_f32, int splits, int64_t part_stride
   if (int rc = check_source(src, src_f32, splits, part_stride, src_stride, q_cols + k_cols, dtype, "tied_prep")) return rc;
   const TiedPrep a{RowSource{src, src_f32, splits, part_stride, src_stride}, bias, wq, factor, q, pool, pool_stride, rms, loc,
                    positions, q_cols, k_cols, q_size, k_size, eps};
-  const int vpt = ((q_cols + k_cols) / 8 + 255) / 256;
-#define SGLK_TP(V) hipLaunchKernelGGL((tied_prep_kernel<T, V>), dim3(M), dim3(256), 0, (hipStream_t)stream, a)
+  const int vecs = (q_cols + k_cols) / 8;
+  const bool wide = M <= 512 && vecs > 256;  // a decode batch: few rows, every piece on a thread of its own
+#define SGLK_TP(BT, V) hipLaunchKernelGGL((tied_prep_kernel<T, BT, V>), dim3(M), dim3(BT), 0, (hipStream_t)stream, a)
   SGLK_DISPATCH_FLOAT(dtype, T, {
-    if (vpt <= 1)
-      SGLK_TP(1);
-    else if (vpt <= 3)
-      SGLK_TP(3);
+    if (vecs <= 256)
+      SGLK_TP(256, 1);
+    else if (wide && vecs <= 768)
+      SGLK_TP(768, 1);
+    else if (wide)
+      SGLK_TP(768, 3);
+    else if (vecs <= 768)
+      SGLK_TP(256, 3);
     else
-      SGLK_TP(8);
+      SGLK_TP(256, 8);
   });
 #undef SGLK_TP
   SGLK_LAUNCH_CHECK();
