@@ -163,8 +163,12 @@ def test_tied_prefill(H_, G, D, dim, buckets, longest, many):
     assert bool((out[:4] == 3.0).all()) and bool((out[:, H_ * D:] == 3.0).all())
 
 
-def test_a_bias_table_too_long_for_the_chip_s_memory():
-    test_tied_prefill(2, 1, 64, 64, 8, 5000, False)
+def test_tied_prefill_with_a_bias_table_beyond_the_lds():
+    from sglang_security_amd.layers.position_bias import bucket_starts
+
+    assert bucket_starts(64, 3000)[-1] > 2048
+    for D, many in ((64, False), (128, True), (192, False)):
+        test_tied_prefill(2, 1, D, D, 64, 3000, many)
 
 
 # ---- gated delta rule -----------------------------------------------------------------------------------------------------
