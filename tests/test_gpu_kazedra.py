@@ -88,7 +88,7 @@ def _tied_want(q, pool, rms, r2t, b, n, rel, longest, sink, first):
     return O.tied_attention(full, k, v, 1.0, rel.double(), longest, sink.double())[first:]
 
 
-TIED = [(6, 2, 32, 24, 10, 40), (8, 1, 64, 64, 16, 120), (2, 2, 96, 80, 4, 9), (40, 2, 128, 128, 32, 300), (3, 1, 192, 192, 2, 40),
+TIED = [(6, 2, 32, 24, 10, 40), (7, 1, 64, 64, 14, 100), (2, 2, 96, 80, 4, 9), (40, 2, 128, 128, 32, 300), (3, 1, 192, 192, 2, 40),
         (18, 1, 64, 50, 64, 128), (2, 1, 256, 256, 12, 64)]
 
 
@@ -195,7 +195,7 @@ def _delta(c, dtype, seed=0, change=None):
 
 
 DELTA = [dict(heads=6, kv_heads=3, dim=20, vdim=12, conv=4), dict(heads=2, kv_heads=2, dim=128, vdim=128, conv=4),
-         dict(heads=4, kv_heads=1, dim=64, vdim=32, conv=2), dict(heads=3, kv_heads=3, dim=96, vdim=80, conv=1),
+         dict(heads=4, kv_heads=1, dim=64, vdim=48, conv=2), dict(heads=3, kv_heads=3, dim=96, vdim=80, conv=1),
          dict(heads=2, kv_heads=1, dim=32, vdim=256, conv=7), dict(heads=1, kv_heads=1, dim=256, vdim=64, conv=3),
          dict(heads=2, kv_heads=1, dim=150, vdim=300, conv=4)]
 
